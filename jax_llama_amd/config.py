@@ -881,3 +881,187 @@ class ZifisunConfig:
 
     def __repr__(self) -> str:
         return f"ZifisunConfig {json.dumps(self.to_dict(), sort_keys=True)}"
+
+
+# -------------------------------------------------------------------------------------
+# Fokisun: normed rotary attention, latent attention and a gated running memory, mixer and feed-forward side by side,
+# layers that read a weighted sum of every earlier layer's result
+# -------------------------------------------------------------------------------------
+@dataclass
+class WholeNormAttentionSpec:
+    """Softmax attention with projection biases, q and k normed over their whole projections, rotary positions on the first
+    ``rot_dims`` numbers of each head (frequencies divided by ``rot_factor``), a sliding window of ``window`` positions (0:
+    none), and, with ``v_mix``, values blended with the first such layer's."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    rot_base: float = 10000.0
+    rot_dims: int = 0
+    rot_factor: float = 1.0
+    window: int = 0
+    v_mix: bool = False
+    type = "attention"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "WholeNormAttentionSpec":
+        heads, dim = int(d["heads"]), int(d["dim"])
+        rot = d.get("rot") or {}
+        window, keep = _mask_from(d.get("mask"))
+        out = cls(heads=heads, kv_heads=int(d.get("kv_heads", heads)), dim=dim, vdim=int(d.get("vdim", dim)),
+                  scale=float(d["scale"]), rot_base=float(rot.get("base", 10000.0)), rot_dims=int(rot.get("dims", 0)),
+                  rot_factor=float((rot.get("scaling") or {}).get("factor", 1.0)), window=window,
+                  v_mix=bool(d.get("v_mix", False)))
+        if out.heads % out.kv_heads:
+            raise ValueError("heads must be divisible by kv_heads")
+        if out.rot_dims % 2 or not 0 <= out.rot_dims <= out.dim or not out.rot_factor > 0.0:
+            raise ValueError("rot.dims must be even and at most dim, rot.scaling.factor positive")
+        if keep:
+            raise ValueError("attention: this mixer's window keeps no first positions")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        out: Dict[str, Any] = dict(heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, scale=self.scale,
+                                   v_mix=self.v_mix)
+        if self.rot_dims:
+            out["rot"] = {"base": self.rot_base, "dims": self.rot_dims}
+            if self.rot_factor != 1.0:
+                out["rot"]["scaling"] = {"factor": self.rot_factor}
+        mask = _mask_to(self.window, 0)
+        if mask:
+            out["mask"] = mask
+        return out
+
+
+@dataclass
+class GatedRunningSpec:
+    """Linear attention whose forget gate also decides what is written: ``heads`` heads of ``dim`` key channels and ``vdim``
+    value numbers."""
+
+    heads: int
+    dim: int
+    vdim: int
+    type = "hgrn2"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "GatedRunningSpec":
+        dim = int(d["dim"])
+        return cls(heads=int(d["heads"]), dim=dim, vdim=int(d.get("vdim", dim)))
+
+    def to_dict(self) -> Dict[str, Any]:
+        return dict(heads=self.heads, dim=self.dim, vdim=self.vdim)
+
+
+@dataclass
+class GatedMoESpec:
+    """Sigmoid-routed mixture of gated experts of width ``ff``: ``top`` of ``experts``, chosen inside the ``keep_groups`` best
+    of ``groups`` equal groups (a group's score: its two largest scores summed), weights normalised and times ``scale``; an
+    optional shared expert of width ``shared_ff``."""
+
+    experts: int
+    top: int
+    groups: int
+    keep_groups: int
+    scale: float
+    ff: int
+    shared_ff: int = 0
+    kind = "moe"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "GatedMoESpec":
+        r = d["router"]
+        gr = r.get("groups") or {}
+        out = cls(experts=int(r["experts"]), top=int(r["top"]), groups=int(gr.get("count", 1)),
+                  keep_groups=int(gr.get("keep", gr.get("count", 1))), scale=float(r.get("scale", 1.0)),
+                  ff=int(d["expert"]["ff"]), shared_ff=int((d.get("shared") or {}).get("ff", 0)))
+        if out.groups < 1 or out.experts % out.groups or not 1 <= out.keep_groups <= out.groups:
+            raise ValueError(f"router: {out.experts} experts do not form {out.groups} equal groups of which "
+                             f"{out.keep_groups} are kept")
+        if not 1 <= out.top <= out.keep_groups * (out.experts // out.groups):
+            raise ValueError(f"router: top {out.top} does not fit the kept groups")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        router: Dict[str, Any] = {"experts": self.experts, "top": self.top, "scale": self.scale}
+        if self.groups > 1:
+            router["groups"] = {"count": self.groups, "keep": self.keep_groups}
+        out: Dict[str, Any] = {"kind": "moe", "expert": {"ff": self.ff}, "router": router}
+        if self.shared_ff:
+            out["shared"] = {"ff": self.shared_ff}
+        return out
+
+
+class FokisunConfig:
+    """Fokisun decoder: ``config.json`` with ``architecture: "Fokisun"``, ``vocab``, ``width``, ``norm.eps``,
+    ``residual_mult``, ``logit_scale`` and a ``layers`` list of ``{type, mixer, mlp}`` entries; ``type`` is ``attention``,
+    ``latent_attention`` or ``hgrn2``, ``mlp`` null, ``{kind: dense, ff}`` or a ``GatedMoESpec`` entry."""
+
+    model_type = "fokisun"
+    architecture = "Fokisun"
+    MIXERS = {"attention": WholeNormAttentionSpec, "latent_attention": RotaryLatentSpec, "hgrn2": GatedRunningSpec}
+
+    def __init__(self, vocab_size: int, hidden_size: int, layers, norm_eps: float = 1e-6, residual_mult: float = 1.0,
+                 logit_scale: float = 1.0, pad_token_id: int = -1, eos_token_id: Optional[int] = None):
+        self.vocab_size = int(vocab_size)
+        self.hidden_size = int(hidden_size)
+        self.layers = list(layers)
+        self.norm_eps = float(norm_eps)
+        self.residual_mult = float(residual_mult)
+        self.logit_scale = float(logit_scale)
+        self.pad_token_id = pad_token_id
+        self.eos_token_id = eos_token_id
+        mixing = [ls.mixer for ls in self.layers if ls.mixer.type == "attention" and ls.mixer.v_mix]
+        if any(m.kv_heads * m.vdim != mixing[0].kv_heads * mixing[0].vdim for m in mixing):
+            raise ValueError("v_mix layers must project equally many values")
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @staticmethod
+    def _ff_from_dict(d: Optional[Dict[str, Any]]):
+        if d is None:
+            return None
+        kind = d.get("kind")
+        if kind == "dense":
+            return DenseFFSpec(ff=int(d["ff"]))
+        if kind == "moe":
+            return GatedMoESpec.from_dict(d)
+        raise ValueError(f"unknown feed-forward kind {kind!r}")
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "FokisunConfig":
+        layers = []
+        for i, e in enumerate(d["layers"]):
+            if e["type"] not in cls.MIXERS:
+                raise ValueError(f"layer {i}: Fokisun has no mixer {e['type']!r}")
+            layers.append(LayerSpec(cls.MIXERS[e["type"]].from_dict(e["mixer"]), cls._ff_from_dict(e.get("mlp"))))
+        return cls(vocab_size=d["vocab"], hidden_size=d["width"], layers=layers, norm_eps=d["norm"]["eps"],
+                   residual_mult=d.get("residual_mult", 1.0), logit_scale=d.get("logit_scale", 1.0),
+                   pad_token_id=d.get("pad_token_id", -1), eos_token_id=d.get("eos_token_id"))
+
+    def to_dict(self) -> Dict[str, Any]:
+        return {"architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size,
+                "norm": {"eps": self.norm_eps}, "residual_mult": self.residual_mult, "logit_scale": self.logit_scale,
+                "layers": [{"type": ls.mixer.type, "mixer": ls.mixer.to_dict(),
+                            "mlp": ls.mlp.to_dict() if ls.mlp is not None else None} for ls in self.layers]}
+
+    def save_pretrained(self, save_directory: str) -> None:
+        os.makedirs(save_directory, exist_ok=True)
+        with open(os.path.join(save_directory, "config.json"), "w") as f:
+            json.dump(self.to_dict(), f, indent=1, sort_keys=True)
+
+    @classmethod
+    def from_pretrained(cls, path: str) -> "FokisunConfig":
+        if os.path.isdir(path):
+            path = os.path.join(path, "config.json")
+        with open(path) as f:
+            return cls.from_dict(json.load(f))
+
+    def __eq__(self, other: object) -> bool:
+        return isinstance(other, FokisunConfig) and self.to_dict() == other.to_dict()
+
+    def __repr__(self) -> str:
+        return f"FokisunConfig {json.dumps(self.to_dict(), sort_keys=True)}"

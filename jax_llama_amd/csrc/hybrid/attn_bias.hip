@@ -17,9 +17,10 @@
 // Sliding windows (window > 0): a query at slot i sees the keys of [max(0, i - window + 1), i] and, with keep_first, the
 // row's first keep_first slots. Every kernel numbers a query's visible keys 0 .. n - 1 (the kept first ones, then the
 // window) and walks that numbering, so hidden keys are never read and the decode splits deal only visible keys; the MFMA
-// kernel walks the kept tiles and then the window's tiles. A gate per (token, head) (sigmoid of a projection column)
-// multiplies the normalised output in the kernels that write it. Values may be the leading columns of wider rows (ldv):
-// a latent cache whose rows carry a rotated key part behind the latent serves as keys (whole row) and values (latent).
+// kernel walks the kept tiles and then the window's tiles. A gate per (token, head) or per output column (sigmoid of
+// projection columns) multiplies the normalised output in the kernels that write it; the output may be a column slice of
+// a wider row, in fp32 or bf16. Values may be the leading columns of wider rows (ldv): a latent cache whose rows carry a
+// rotated key part behind the latent serves as keys (whole row) and values (latent).
 #include "hy_util.h"
 #include "hybrid.h"
 
@@ -106,7 +107,15 @@ JLA_DEV AbSpan ab_span(const AttnBias& p, int qi) {
   return sp;
 }
 JLA_DEV int ab_key(const AbSpan& sp, int v) { return v < sp.kf ? v : sp.lo + (v - sp.kf); }
-JLA_DEV float ab_gate(const AttnBias& p, size_t m, int h) { return p.gate ? hy_sigmoid(p.gate[m * p.ldg + h]) : 1.f; }
+// gate of column c of head h: one per head, or one per column
+JLA_DEV float ab_gate(const AttnBias& p, size_t m, int h, int c) {
+  return p.gate ? hy_sigmoid(p.gate[m * p.ldg + (p.gate_cols ? h * p.vdim + c : h)]) : 1.f;
+}
+JLA_DEV void ab_out(const AttnBias& p, size_t m, int h, int c, float v) {
+  const size_t at = m * p.ldo + (size_t)h * p.vdim + c;
+  if (p.out_bf16) reinterpret_cast<bf16_t*>(p.out)[at] = f2bf(v);
+  else reinterpret_cast<float*>(p.out)[at] = v;
+}
 
 // One wave: visible keys number [j_lo, j_hi) of query (b, h) at slot qi (span); returns the running max m, sum l and
 // unnormalised acc. with_sink: the wave whose keys start the row also counts the head's sink.
@@ -202,12 +211,12 @@ __global__ void __launch_bounds__(256) attn_bias_prefill_kernel(AttnBias p) {
   float m_run, l_run, acc[VREG];
   const AbSpan span = ab_span(p, qi);
   ab_wave<CT, VREG>(p, qs, b, h, qi, span, 0, span.n, true, m_run, l_run, acc);
-  float* o = p.out + ((size_t)b * p.S + s) * (p.H * p.vdim) + (size_t)h * p.vdim;
-  const float inv = ab_gate(p, (size_t)b * p.S + s, h) / l_run;
+  const size_t m = (size_t)b * p.S + s;
+  const float inv = 1.f / l_run;
 #pragma unroll
   for (int i = 0; i < VREG; ++i) {
     const int c = lane + 64 * i;
-    if (c < p.vdim) o[c] = acc[i] * inv;
+    if (c < p.vdim) ab_out(p, m, h, c, acc[i] * (inv * ab_gate(p, m, h, c)));
   }
 }
 
@@ -443,14 +452,14 @@ __global__ void __launch_bounds__(64) attn_bias_merge_kernel(AttnBias p) {
   const float m = wave_max(ls > 0.f ? ms : -INFINITY);
   const float wt = ls > 0.f ? expf(ms - m) : 0.f;  // weight of this lane's split
   const float l = wave_sum(ls * wt);
-  float* o = p.out + (size_t)b * (p.H * p.vdim) + (size_t)h * p.vdim;
+  const float gt = ab_gate(p, b, h, c);
   float a = 0.f;
 #pragma unroll
   for (int sp = 0; sp < 64; ++sp) {  // (a split without keys holds zeros and has weight 0)
     const float ws = __shfl(wt, sp, 64);
     a = fmaf(part[sp], sp < p.splits ? ws : 0.f, a);
   }
-  if (c0 + lane < p.vdim) o[c] = a / l * ab_gate(p, b, h);
+  if (c0 + lane < p.vdim) ab_out(p, b, h, c, a / l * gt);
 }
 
 // ---- MFMA flash prefill (bf16 caches) ----------------------------------------------------------------------------------
@@ -619,14 +628,23 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
   }
   l_run += __shfl_xor(l_run, 32, 64);
   if (s0 + ql >= p.S) return;
-  const float inv = ab_gate(p, (size_t)b * p.S + s0 + ql, h) / l_run;
-  float* out = p.out + ((size_t)b * p.S + s0 + ql) * (p.H * vdim) + (size_t)h * vdim;
+  const size_t m = (size_t)b * p.S + s0 + ql;
+  const float inv = p.gate && !p.gate_cols ? ab_gate(p, m, h, 0) / l_run : 1.f / l_run;
+  const size_t at = m * p.ldo + (size_t)h * vdim;
+  const float* gt = p.gate && p.gate_cols ? p.gate + m * p.ldg + (size_t)h * vdim : nullptr;
 #pragma unroll
   for (int v = 0; v < VT; ++v)
 #pragma unroll
     for (int r = 0; r < 16; r += 4) {  // rows (value columns) (r & 3) + 8 (r >> 2) + 4 hi: runs of four
-      const float4 w = {o[v][r] * inv, o[v][r + 1] * inv, o[v][r + 2] * inv, o[v][r + 3] * inv};
-      *reinterpret_cast<float4*>(out + 32 * v + 8 * (r >> 2) + 4 * hi) = w;
+      const int c = 32 * v + 8 * (r >> 2) + 4 * hi;
+      float f[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) f[k] = o[v][r + k] * inv * (gt ? hy_sigmoid(gt[c + k]) : 1.f);
+      if (p.out_bf16)
+        *reinterpret_cast<uint2*>(reinterpret_cast<bf16_t*>(p.out) + at + c) =
+            uint2{(uint32_t)f2bf(f[0]) | (uint32_t)f2bf(f[1]) << 16, (uint32_t)f2bf(f[2]) | (uint32_t)f2bf(f[3]) << 16};
+      else
+        *reinterpret_cast<float4*>(reinterpret_cast<float*>(p.out) + at + c) = float4{f[0], f[1], f[2], f[3]};
     }
 }
 
@@ -640,10 +658,15 @@ static int am_launch(const AttnBias& p, bf16_t* vt, int Tp, hipStream_t s) {
   return 0;
 }
 
+// key widths the flash kernel is instantiated for (beside 64 and 128: plain numbers plus a rotated part of 16 .. 64)
+static bool am_key_width(int dim) {
+  return dim == 64 || dim == 80 || dim == 96 || dim == 128 || dim == 160 || dim == 192;
+}
+
 // bytes of the transposed-value workspace the MFMA prefill needs, 0 when the shape goes to the plain kernel
 long long hy_attn_prefill_ws_bytes(int B, int S, int G, int dim, int vdim, int T, int cbf16) {
   if (!cbf16 || S < 2) return 0;
-  if (!((dim == 64 || dim == 128) && (vdim == 64 || vdim == 128))) return 0;
+  if (!am_key_width(dim) || !(vdim == 64 || vdim == 128)) return 0;
   if ((long long)B * G > 65535) return 0;
   return (long long)B * G * vdim * ((T + 31) / 32 * 32) * 2;
 }
@@ -681,7 +704,7 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
   if (p.dim < 1 || p.dim > AB_MAX_DIM || p.vdim < 1 || p.vdim > 64 * AB_MAX_VREG) return -2;
   if (p.bias && p.nbias < 1) return -3;
   if (p.chunk < 0 || p.window < 0 || p.keep_first < 0 || (p.chunk > 0 && p.window > 0)) return -7;
-  if (p.ldv < p.vdim || (p.gate && p.ldg < p.H)) return -8;
+  if (p.ldv < p.vdim || (p.gate && p.ldg < (p.gate_cols ? p.H * p.vdim : p.H)) || p.ldo < p.H * p.vdim) return -8;
   if (p.B == 0) return 0;
   if (p.H > 65535 || p.B > 65535) return -4;
   if (p.S == 1) {
@@ -705,13 +728,24 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
     JLA_CHECK_LAUNCH();
     return 0;
   }
-  if (p.vt_ws && p.ldv == p.vdim && hy_attn_prefill_ws_bytes(p.B, p.S, p.G, p.dim, p.vdim, p.T, p.cbf16) > 0) {
+  // (the flash kernel stores four columns at a time)
+  if (p.vt_ws && p.ldv == p.vdim && p.ldo % 4 == 0 && ((uintptr_t)p.out & (p.out_bf16 ? 7 : 15)) == 0 &&
+      hy_attn_prefill_ws_bytes(p.B, p.S, p.G, p.dim, p.vdim, p.T, p.cbf16) > 0) {
     const int Tp = (p.T + 31) / 32 * 32;
     bf16_t* vt = reinterpret_cast<bf16_t*>(p.vt_ws);
-    if (p.dim == 64 && p.vdim == 64) return am_launch<4, 2>(p, vt, Tp, s);
-    if (p.dim == 64 && p.vdim == 128) return am_launch<4, 4>(p, vt, Tp, s);
-    if (p.dim == 128 && p.vdim == 64) return am_launch<8, 2>(p, vt, Tp, s);
-    return am_launch<8, 4>(p, vt, Tp, s);
+#define AM_CASE(DK)                                               \
+  case 16 * DK:                                                   \
+    return p.vdim == 64 ? am_launch<DK, 2>(p, vt, Tp, s) : am_launch<DK, 4>(p, vt, Tp, s)
+    switch (p.dim) {
+      AM_CASE(4);
+      AM_CASE(5);
+      AM_CASE(6);
+      AM_CASE(8);
+      AM_CASE(10);
+      AM_CASE(12);
+    }
+#undef AM_CASE
+    return -9;
   }
   dim3 grid((p.S + 3) / 4, p.H, p.B);
   AB_BY_VREG(attn_bias_prefill_kernel, grid, 256);

@@ -86,7 +86,7 @@ void linear_rows(Tensor a, OptT a_idx, Tensor w, Tensor out, OptT dst_idx, OptT 
   p.E = w.dim() == 3 ? w.size(0) : 1;
   const int64_t Nw = w.size(-2);
   p.K = w.size(-1);
-  check(act >= jla::HY_ACT_NONE && act <= jla::HY_ACT_SOFTCAP, "linear_rows: unknown activation");
+  check(act >= jla::HY_ACT_NONE && act <= jla::HY_ACT_GELU_GLU, "linear_rows: unknown activation");
   const bool gated = jla::hy_act_gated(act);
   check(!gated || Nw % 2 == 0, "linear_rows: a gated activation needs gate and up rows");
   p.N = gated ? Nw / 2 : Nw;
@@ -157,7 +157,8 @@ void route_topk(Tensor z, int64_t E, int64_t top, Tensor row_expert, Tensor row_
 }
 
 void route_grouped(Tensor z, OptT correction, int64_t E, int64_t top, int64_t groups, int64_t keep, Tensor row_expert,
-                   Tensor row_tok, Tensor row_w, OptT sort_tok, OptT sort_dst, OptT sort_w, OptT offs) {
+                   Tensor row_tok, Tensor row_w, OptT sort_tok, OptT sort_dst, OptT sort_w, OptT offs, bool sigmoid,
+                   int64_t group_top, bool normalise, double w_scale) {
   check(z.dim() == 2 && z.size(1) >= E && top >= 1 && top <= E, "route_grouped: z is [M, >= E], 1 <= top <= E");
   int ldz = 0;
   const float* zp = rows2d(z, "z", z.size(1), &ldz);
@@ -169,8 +170,9 @@ void route_grouped(Tensor z, OptT correction, int64_t E, int64_t top, int64_t gr
   check(sorted == sort_dst.has_value() && sorted == sort_w.has_value() && sorted == offs.has_value(),
         "route_grouped: the sorted outputs come together");
   check(!sorted || sort_w->numel() >= R, "route_grouped: weight outputs hold R numbers");
-  rc(jla::hy_route_grouped(zp, ldz, correction.has_value() ? f32(*correction, "correction") : nullptr, M, top, E, groups,
-                           keep, i32w(row_expert, "row_expert", R), i32w(row_tok, "row_tok", R), f32w(row_w, "row_w"),
+  rc(jla::hy_route_grouped(zp, ldz, correction.has_value() ? f32(*correction, "correction") : nullptr, M, top, E,
+                           jla::RouteRule{(int)groups, (int)keep, (int)group_top, sigmoid, normalise, (float)w_scale},
+                           i32w(row_expert, "row_expert", R), i32w(row_tok, "row_tok", R), f32w(row_w, "row_w"),
                            sorted ? i32w(*sort_tok, "sort_tok", R) : nullptr,
                            sorted ? i32w(*sort_dst, "sort_dst", R) : nullptr, sorted ? f32w(*sort_w, "sort_w") : nullptr,
                            sorted ? i32w(*offs, "offs", E + 1) : nullptr, stream()),
@@ -268,6 +270,71 @@ void gelu_gate_rows(Tensor gp, Tensor ids, Tensor table, int64_t col0, Tensor g)
      "gelu_gate_rows");
 }
 
+void* slice2d_any(const Tensor& t, const char* name, int64_t rows, int64_t cols, int* ld, int* bf);
+
+void glu_rows(Tensor gu, Tensor out, int64_t act, double limit, double alpha) {
+  check(gu.dim() == 2 && out.dim() == 2 && gu.size(1) == 2 * out.size(1) && jla::hy_act_gated(act),
+        "glu_rows: gu is [M, 2F], out [M, F], a gated activation");
+  int ldo = 0, bf = 0;
+  void* op = slice2d_any(out, "out", gu.size(0), out.size(1), &ldo, &bf);
+  rc(jla::hy_glu_rows(f32(gu, "gu"), gu.size(0), out.size(1), act, limit, alpha, op, bf, ldo, stream()), "glu_rows");
+}
+
+// fp32 or bf16 dense [M, D] output
+void* rows_out(const Tensor& h, const char* name, int64_t n, int* bf) {
+  *bf = wtype(h, name);
+  check(h.numel() == n, "an output row tensor has the wrong size");
+  return h.data_ptr();
+}
+
+void squash_rows(Tensor x, Tensor alpha, Tensor w, Tensor b, Tensor h) {
+  check(x.dim() == 2, "squash_rows: x is [M, D]");
+  const int64_t M = x.size(0), D = x.size(1);
+  check(alpha.numel() == 1 && w.numel() == D && b.numel() == D, "squash_rows: alpha is one number, w and b are [D]");
+  int bf = 0;
+  void* hp = rows_out(h, "h", M * D, &bf);
+  rc(jla::hy_squash_rows(f32(x, "x"), M, D, f32(alpha, "alpha"), f32(w, "w"), f32(b, "b"), hp, bf, stream()),
+     "squash_rows");
+}
+
+void depth_update(Tensor hist, int64_t i, bool store, Tensor x, Tensor x_out, double mult, Tensor y, OptT bias, OptT ye,
+                  int64_t nsum, OptT row_w, Tensor coef, OptT alpha, OptT w, OptT b, OptT h) {
+  jla::DepthUpdate p{};
+  check(hist.dim() == 3 && i >= 0 && i + (store ? 1 : 0) < hist.size(0), "depth_update: hist is [planes, M, D], planes past i");
+  p.M = hist.size(1); p.D = hist.size(2);
+  const int64_t md = (int64_t)p.M * p.D;
+  p.hist = f32w(hist, "hist");
+  p.i = i; p.store = store;
+  check(x.numel() == md && x_out.numel() == md && y.numel() == md, "depth_update: x, x_out and y are [M, D]");
+  p.x = f32(x, "x");
+  p.x_out = f32w(x_out, "x_out");
+  p.mult = mult;
+  p.y = f32(y, "y");
+  if (bias.has_value()) {
+    check(bias->numel() == p.D, "depth_update: bias is [D]");
+    p.bias = f32(*bias, "bias");
+  }
+  if (ye.has_value()) {
+    check(row_w.has_value() && nsum >= 1 && ye->numel() == md * nsum && row_w->numel() >= p.M * nsum,
+          "depth_update: ye is [M * nsum, D], row_w [M * nsum]");
+    p.ye = f32(*ye, "ye");
+    p.row_w = f32(*row_w, "row_w");
+    p.nsum = nsum;
+  }
+  check(coef.numel() == i + 2, "depth_update: coef is [i + 2]");
+  p.coef = f32(coef, "coef");
+  if (h.has_value()) {
+    check(alpha.has_value() && w.has_value() && b.has_value() && alpha->numel() == 1 && w->numel() == p.D &&
+              b->numel() == p.D,
+          "depth_update: the norm's alpha is one number, w and b are [D]");
+    p.alpha = f32(*alpha, "alpha");
+    p.w = f32(*w, "w");
+    p.b = f32(*b, "b");
+    p.h = rows_out(*h, "h", md, &p.h_bf16);
+  }
+  rc(jla::hy_depth_update(p, stream()), "depth_update");
+}
+
 void attn_prep(Tensor proj, Tensor positions, Tensor slot, int64_t B, int64_t S, int64_t H, int64_t G, int64_t dim,
                int64_t vdim, OptT kc, OptT vc, Tensor q, double eps, double temp_coef, int64_t temp_every, OptT q_w, OptT k_w,
                bool norm_v) {
@@ -311,8 +378,9 @@ void attn_prep(Tensor proj, Tensor positions, Tensor slot, int64_t B, int64_t S,
 const double* f64(const Tensor& t, const char* name);
 
 void latent_prep(Tensor proj, int64_t col0, Tensor w, Tensor slot, int64_t B, int64_t S, Tensor cache, double eps,
-                 OptT q, int64_t q_col0, OptT q_norm_w, OptT rot_freq, OptT positions) {
+                 OptT q, int64_t q_col0, OptT q_norm_w, OptT rot_freq, OptT positions, bool rot_halves) {
   jla::LatentPrep p{};
+  p.rot_halves = rot_halves;
   check(proj.dim() == 2 && proj.size(0) == B * S && proj.scalar_type() == torch::kFloat32 && proj.is_cuda() &&
             proj.stride(1) == 1,
         "latent_prep: proj is a float32 [B * S, cols] GPU view with unit inner stride");
@@ -339,7 +407,7 @@ void latent_prep(Tensor proj, int64_t col0, Tensor w, Tensor slot, int64_t B, in
   if (q.has_value()) {
     check(q->dim() == 2 && q->size(0) == B * S && q_col0 >= 0 && q_col0 + q->size(1) <= proj.size(1),
           "latent_prep: q is [B * S, q_cols]");
-    p.q = f32w(*q, "q");
+    p.q = rows_out(*q, "q", q->numel(), &p.q_bf16);
     p.q_cols = q->size(1);
     p.q_col0 = q_col0;
     if (q_norm_w.has_value()) {
@@ -358,7 +426,7 @@ int64_t attn_prefill_ws_bytes(int64_t B, int64_t S, int64_t G, int64_t dim, int6
 
 void attn_bias(Tensor q, Tensor kc, Tensor vc, Tensor slot, double scale, double softcap, OptT bias, Tensor out,
                int64_t t_cap, OptT ws, int64_t splits, OptT vt_ws, OptT sink, int64_t chunk, OptT head_scale, int64_t window,
-               int64_t keep_first, OptT gate, c10::optional<int64_t> vdim) {
+               int64_t keep_first, OptT gate, c10::optional<int64_t> vdim, bool gate_cols) {
   jla::AttnBias p{};
   check(q.dim() == 4, "attn_bias: q is [B, S, H, dim]");
   p.B = q.size(0); p.S = q.size(1); p.H = q.size(2); p.dim = q.size(3);
@@ -376,7 +444,10 @@ void attn_bias(Tensor q, Tensor kc, Tensor vc, Tensor slot, double scale, double
   p.window = window;
   p.keep_first = keep_first;
   if (gate.has_value()) {
-    check(gate->dim() == 2 && gate->size(0) == (int64_t)p.B * p.S && gate->size(1) >= p.H, "attn_bias: gate is [B * S, >= H]");
+    p.gate_cols = gate_cols;
+    check(gate->dim() == 2 && gate->size(0) == (int64_t)p.B * p.S &&
+              gate->size(1) >= (gate_cols ? (int64_t)p.H * p.vdim : (int64_t)p.H),
+          "attn_bias: gate is [B * S, >= H], with gate_cols [B * S, >= H * vdim]");
     p.gate = rows2d(*gate, "gate", gate->size(1), &p.ldg);
   }
   p.kc = kc.data_ptr();
@@ -399,8 +470,7 @@ void attn_bias(Tensor q, Tensor kc, Tensor vc, Tensor slot, double scale, double
     check(head_scale->numel() == p.H, "attn_bias: head_scale is [H]");
     p.head_scale = f32(*head_scale, "head_scale");
   }
-  check(out.numel() == (int64_t)p.B * p.S * p.H * p.vdim, "attn_bias: out shape");
-  p.out = f32w(out, "out");
+  p.out = slice2d_any(out, "out", (int64_t)p.B * p.S, (int64_t)p.H * p.vdim, &p.ldo, &p.out_bf16);
   p.t_cap = std::min<int64_t>(t_cap, p.T);
   p.splits = splits;
   if (p.S == 1) {
@@ -486,6 +556,18 @@ float* slice2d(const Tensor& t, const char* name, int64_t rows, int64_t cols, in
   return reinterpret_cast<float*>(t.data_ptr());
 }
 
+// the same, float32 or bfloat16 (*bf = 1)
+void* slice2d_any(const Tensor& t, const char* name, int64_t rows, int64_t cols, int* ld, int* bf) {
+  TORCH_CHECK(t.is_cuda() && (t.scalar_type() == torch::kFloat32 || t.scalar_type() == torch::kBFloat16) &&
+                  t.dim() == 2 && (t.size(1) <= 1 || t.stride(1) == 1) && t.size(0) == rows && t.size(1) == cols &&
+                  (rows <= 1 || t.stride(0) >= cols),
+              "jax_llama_amd._C_hybrid: ", name, " must be a float32 / bfloat16 [", rows, ", ", cols,
+              "] GPU view with unit inner stride");
+  *ld = rows > 1 ? (int)t.stride(0) : (int)cols;
+  *bf = t.scalar_type() == torch::kBFloat16;
+  return t.data_ptr();
+}
+
 // a [M, H, n] float32 view whose heads are adjacent (stride(1) == n, unit inner stride): rows may be strided
 const float* heads3d(const Tensor& t, const char* name, int64_t M, int64_t H, int64_t n, int* ld) {
   TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kFloat32 && t.dim() == 3 && t.size(0) == M && t.size(1) == H &&
@@ -502,19 +584,22 @@ const double* f64(const Tensor& t, const char* name) {
   return reinterpret_cast<const double*>(t.data_ptr());
 }
 
-void gated_rmsnorm(Tensor o, Tensor gate, Tensor w, double eps, Tensor out, int64_t H, int64_t vdim, int64_t gate_act,
+void gated_rmsnorm(Tensor o, OptT gate, Tensor w, double eps, Tensor out, int64_t H, int64_t vdim, int64_t gate_act,
                    OptT denom_floor, double gain) {
   jla::GatedNorm p{};
   const int64_t ov = denom_floor.has_value() ? vdim + 1 : vdim;
   const int64_t M = o.numel() / (H * ov);
   check(o.numel() == M * H * ov && (w.numel() == vdim || w.numel() == H * vdim), "gated_rmsnorm shapes");
-  check(gate.dim() == 2 && gate.size(0) == M, "gated_rmsnorm: gate rows");
+  check(gate.has_value() == (gate_act != 2), "gated_rmsnorm: gate_act 2 has no gate, the others need one");
   p.o = f32(o, "o");
-  p.gate = rows2d(gate, "gate", H * vdim, &p.ldg);
+  if (gate.has_value()) {
+    check(gate->dim() == 2 && gate->size(0) == M, "gated_rmsnorm: gate rows");
+    p.gate = rows2d(*gate, "gate", H * vdim, &p.ldg);
+  }
   p.w = f32(w, "w");
   p.w_heads = w.numel() != vdim || H == 1;
   p.eps = eps;
-  p.out = slice2d(out, "out", M, H * vdim, &p.ldo);
+  p.out = slice2d_any(out, "out", M, H * vdim, &p.ldo, &p.out_bf16);
   p.M = M; p.H = H; p.vdim = vdim;
   p.gate_act = gate_act;
   if (denom_floor.has_value()) {
@@ -559,6 +644,58 @@ void rope_prep(Tensor proj, OptT bias, Tensor positions, Tensor slot, int64_t B,
   rc(jla::hy_rope_prep(p, stream()), "rope_prep");
 }
 
+void qkv_prep(Tensor proj, OptT bias, OptT q_w, OptT k_w, double eps, Tensor positions, Tensor slot, int64_t B, int64_t S,
+              int64_t H, int64_t G, int64_t dim, int64_t vdim, Tensor kc, Tensor vc, Tensor q, OptT freq, bool halves,
+              OptT v_prev, OptT lambda, OptT v_out) {
+  jla::QkvPrep p{};
+  const int64_t cols = (H + G) * dim + G * vdim;
+  check(proj.dim() == 2 && proj.size(0) == B * S && proj.size(1) >= cols, "qkv_prep: proj is [B * S, >= q | k | v columns]");
+  p.proj = rows2d(proj, "proj", proj.size(1), &p.ld);
+  if (bias.has_value()) {
+    check(bias->numel() == cols, "qkv_prep: one bias per projection column");
+    p.bias = f32(*bias, "bias");
+  }
+  if (q_w.has_value()) {
+    check(q_w->numel() == H * dim, "qkv_prep: q_w is [H * dim]");
+    p.q_w = f32(*q_w, "q_w");
+  }
+  if (k_w.has_value()) {
+    check(k_w->numel() == G * dim, "qkv_prep: k_w is [G * dim]");
+    p.k_w = f32(*k_w, "k_w");
+  }
+  p.eps = eps;
+  p.positions = i32(positions, "positions", B * S);
+  p.slot = i32(slot, "slot", 1);
+  p.B = B; p.S = S; p.H = H; p.G = G; p.dim = dim; p.vdim = vdim;
+  p.cbf16 = wtype(kc, "k cache");
+  check(wtype(vc, "v cache") == p.cbf16, "qkv_prep: cache dtypes differ");
+  check(kc.dim() == 4 && kc.size(0) == B && kc.size(1) == G && kc.size(3) == dim, "qkv_prep: k cache shape");
+  p.T = kc.size(2);
+  check(vc.dim() == 4 && vc.size(0) == B && vc.size(1) == G && vc.size(2) == p.T && vc.size(3) == vdim,
+        "qkv_prep: v cache shape");
+  p.kc = kc.data_ptr();
+  p.vc = vc.data_ptr();
+  check(q.numel() == B * S * H * dim, "qkv_prep: q shape");
+  p.q = f32w(q, "q");
+  if (freq.has_value() && freq->numel() > 0) {
+    p.half = freq->numel();
+    check(2 * p.half <= dim, "qkv_prep: more rotated numbers than a head holds");
+    p.freq = f64(*freq, "freq");
+  }
+  p.halves = halves;
+  if (v_prev.has_value()) {
+    check(v_prev->numel() == B * S * G * vdim && lambda.has_value() && lambda->numel() == 1,
+          "qkv_prep: v_prev is [B * S, G * vdim], lambda one number");
+    p.v_prev = f32(*v_prev, "v_prev");
+    p.lambda = f32(*lambda, "lambda");
+  }
+  if (v_out.has_value()) {
+    check(v_out->numel() == B * S * G * vdim, "qkv_prep: v_out is [B * S, G * vdim]");
+    p.v_out = f32w(*v_out, "v_out");
+  }
+  rc(jla::hy_qkv_prep(p, stream()), "qkv_prep");
+}
+
 void rotate_heads(Tensor a, Tensor positions, OptT freq, int64_t H, double sign, double gain, Tensor out, int64_t offset,
                   bool interleaved) {
   check(a.dim() == 2 && a.size(1) % H == 0, "rotate_heads: a is [M, H * n]");
@@ -601,7 +738,7 @@ void mlstm_prep(Tensor proj, int64_t col_i, int64_t col_f, Tensor gate_bias, dou
 void lin_scan(int64_t mode, Tensor q, Tensor k, Tensor v, Tensor decay, OptT write, OptT w0, OptT u, Tensor state,
               Tensor o, int64_t B, int64_t S, double q_scale, int64_t nseg, int64_t seg_len, OptT seg_ws) {
   jla::LinScan p{};
-  check(mode == 0 || mode == 1, "lin_scan: mode");
+  check(mode >= 0 && mode <= 2, "lin_scan: mode");
   check(q.dim() == 3 && v.dim() == 3, "lin_scan: q, k are [M, H, dim], v is [M, H, vdim]");
   const int64_t M = B * S, H = q.size(1), dim = q.size(2), vdim = v.size(2);
   const int64_t cols = mode == 0 ? vdim + 1 : vdim;
@@ -614,7 +751,7 @@ void lin_scan(int64_t mode, Tensor q, Tensor k, Tensor v, Tensor decay, OptT wri
     p.decay = f32(decay, "keep");
     p.write = f32(*write, "write");
   } else {
-    p.decay = heads3d(decay, "decay", M, H, dim, &p.ldd);
+    if (mode == 1) p.decay = heads3d(decay, "decay", M, H, dim, &p.ldd);
     check(w0.has_value() && u.has_value() && w0->numel() == H * dim && u->numel() == H * dim, "lin_scan: w0, u are [H, dim]");
     p.w0 = f32(*w0, "w0");
     p.u = f32(*u, "u");
@@ -628,7 +765,7 @@ void lin_scan(int64_t mode, Tensor q, Tensor k, Tensor v, Tensor decay, OptT wri
   p.nseg = nseg;
   p.seg_len = seg_len;
   if (nseg > 1) {
-    const int64_t ns = B * nseg * H * dim * cols, nd = B * nseg * H * (mode == 1 ? dim : 1);
+    const int64_t ns = B * nseg * H * dim * cols, nd = B * nseg * H * (mode != 0 ? dim : 1);
     check(seg_ws.has_value() && seg_ws->numel() >= ns + nd, "lin_scan: segment workspace");
     p.seg_state = f32w(*seg_ws, "seg_ws");
     p.seg_decay = p.seg_state + ns;
@@ -642,7 +779,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.attr("GEMV_MAX_R") = jla::HY_GEMV_MAX_R;
   m.def("embed_rows", &embed_rows, py::arg("ids"), py::arg("table"), py::arg("col0"), py::arg("out"), py::arg("scale"),
         py::arg("copies") = 1);
-  m.def("route_grouped", &route_grouped);
+  m.def("route_grouped", &route_grouped, py::arg("z"), py::arg("correction"), py::arg("E"), py::arg("top"),
+        py::arg("groups"), py::arg("keep"), py::arg("row_expert"), py::arg("row_tok"), py::arg("row_w"),
+        py::arg("sort_tok"), py::arg("sort_dst"), py::arg("sort_w"), py::arg("offs"), py::arg("sigmoid") = false,
+        py::arg("group_top") = 1, py::arg("normalise") = false, py::arg("w_scale") = 1.0);
   m.def("hc_update", &hc_update);
   m.def("linear_rows", &linear_rows, py::arg("a"), py::arg("a_idx"), py::arg("w"), py::arg("out"), py::arg("dst_idx"),
         py::arg("offs"), py::arg("row_expert"), py::arg("R"), py::arg("act"), py::arg("act_limit"), py::arg("act_alpha"),
@@ -653,7 +793,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("dense_is_gemv", &dense_is_gemv);
   m.def("latent_prep", &latent_prep, py::arg("proj"), py::arg("col0"), py::arg("w"), py::arg("slot"), py::arg("B"),
         py::arg("S"), py::arg("cache"), py::arg("eps"), py::arg("q"), py::arg("q_col0") = 0,
-        py::arg("q_norm_w") = py::none(), py::arg("rot_freq") = py::none(), py::arg("positions") = py::none());
+        py::arg("q_norm_w") = py::none(), py::arg("rot_freq") = py::none(), py::arg("positions") = py::none(),
+        py::arg("rot_halves") = false);
   m.attr("ACT_NONE") = (int)jla::HY_ACT_NONE;
   m.attr("ACT_RELU2") = (int)jla::HY_ACT_RELU2;
   m.attr("ACT_SWIGLU") = (int)jla::HY_ACT_SWIGLU;
@@ -670,7 +811,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_bias", &attn_bias, py::arg("q"), py::arg("kc"), py::arg("vc"), py::arg("slot"), py::arg("scale"),
         py::arg("softcap"), py::arg("bias"), py::arg("out"), py::arg("t_cap"), py::arg("ws"), py::arg("splits"),
         py::arg("vt_ws"), py::arg("sink"), py::arg("chunk") = 0, py::arg("head_scale") = py::none(),
-        py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("gate") = py::none(), py::arg("vdim") = py::none());
+        py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("gate") = py::none(), py::arg("vdim") = py::none(),
+        py::arg("gate_cols") = false);
   m.def("attn_prefill_ws_bytes", &attn_prefill_ws_bytes);
   m.def("delta_prep", &delta_prep);
   m.def("conv_state_update", &conv_state_update);
@@ -680,6 +822,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("gain") = 1.0);
   m.attr("ACT_SOFTCAP") = (int)jla::HY_ACT_SOFTCAP;
   m.def("rope_prep", &rope_prep);
+  m.def("qkv_prep", &qkv_prep, py::arg("proj"), py::arg("bias"), py::arg("q_w"), py::arg("k_w"), py::arg("eps"),
+        py::arg("positions"), py::arg("slot"), py::arg("B"), py::arg("S"), py::arg("H"), py::arg("G"), py::arg("dim"),
+        py::arg("vdim"), py::arg("kc"), py::arg("vc"), py::arg("q"), py::arg("freq"), py::arg("halves") = false,
+        py::arg("v_prev") = py::none(), py::arg("lambda_") = py::none(), py::arg("v_out") = py::none());
+  m.def("glu_rows", &glu_rows);
+  m.def("squash_rows", &squash_rows);
+  m.def("depth_update", &depth_update);
   m.def("rotate_heads", &rotate_heads, py::arg("a"), py::arg("positions"), py::arg("freq"), py::arg("H"), py::arg("sign"),
         py::arg("gain"), py::arg("out"), py::arg("offset") = 0, py::arg("interleaved") = false);
   m.def("token_shift", &token_shift);

@@ -266,18 +266,21 @@ __global__ void __launch_bounds__(256) gated_rmsnorm_kernel(GatedNorm p) {
   }
   ss = wave_sum(ss);
   const float sc = 1.f / sqrtf(ss / (float)vdim + p.eps);
-  const float* gr = p.gate + (size_t)m * p.ldg + (size_t)h * vdim;
+  const float* gr = p.gate_act == 2 ? nullptr : p.gate + (size_t)m * p.ldg + (size_t)h * vdim;
   const float* w = p.w + (p.w_heads ? (size_t)h * vdim : 0);
-  float* dst = p.out + (size_t)m * p.ldo + (size_t)h * vdim;
+  const size_t at = (size_t)m * p.ldo + (size_t)h * vdim;
   for (int d = lane; d < vdim; d += 64) {
-    const float g = p.gate_act == 1 ? hy_sigmoid(gr[d]) : hy_silu(gr[d]);
-    dst[d] = (x[d] * pre) * sc * w[d] * g * p.gain;
+    const float g = p.gate_act == 2 ? 1.f : (p.gate_act == 1 ? hy_sigmoid(gr[d]) : hy_silu(gr[d]));
+    const float v = (x[d] * pre) * sc * w[d] * g * p.gain;
+    if (p.out_bf16) reinterpret_cast<bf16_t*>(p.out)[at + d] = f2bf(v);
+    else reinterpret_cast<float*>(p.out)[at + d] = v;
   }
 }
 
 int hy_gated_rmsnorm(const GatedNorm& p, hipStream_t s) {
-  if (p.M < 0 || p.H < 1 || p.vdim < 1 || p.ldg < p.H * p.vdim || p.ldo < p.H * p.vdim) return -1;
-  if (p.gate_act != 0 && p.gate_act != 1) return -3;
+  if (p.M < 0 || p.H < 1 || p.vdim < 1 || p.ldo < p.H * p.vdim) return -1;
+  if (p.gate_act < 0 || p.gate_act > 2) return -3;
+  if (p.gate_act != 2 && (!p.gate || p.ldg < p.H * p.vdim)) return -1;
   if (p.M == 0) return 0;
   if ((p.H + 3) / 4 > 65535) return -2;
   gated_rmsnorm_kernel<<<dim3(p.M, (p.H + 3) / 4), 256, 0, s>>>(p);

@@ -25,6 +25,9 @@ JLA_DEV void hy_load8(const bf16_t* p, int n, float* f) {
 
 JLA_DEV float hy_silu(float x) { return x / (1.f + expf(-x)); }
 JLA_DEV float hy_sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+JLA_DEV float hy_gelu_tanh(float z) {
+  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
 JLA_DEV float hy_softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
 }  // namespace jla

@@ -24,6 +24,7 @@ enum RowAct {
   HY_ACT_SWIGLU = 2,      // out = silu(g) * u
   HY_ACT_CLAMP_GLU = 3,   // g = min(g, limit), u = clamp(u, -limit, limit): out = g * sigmoid(alpha g) * (u + 1)
   HY_ACT_SOFTCAP = 4,     // out = limit * tanh(y / limit)   (limit = 1: tanh)
+  HY_ACT_GELU_GLU = 5,    // out = gelu_tanh(g) * u
 };
 
 struct RowLinear {
@@ -53,7 +54,9 @@ struct RowLinear {
   float act_alpha;
   int add_out;           // out += act(...) instead of out = (fp32 outputs): a residual add in the epilogue
 };
-inline bool hy_act_gated(int act) { return act == HY_ACT_SWIGLU || act == HY_ACT_CLAMP_GLU; }
+inline bool hy_act_gated(int act) {
+  return act == HY_ACT_SWIGLU || act == HY_ACT_CLAMP_GLU || act == HY_ACT_GELU_GLU;
+}
 // R <= HY_GEMV_MAX_R and (offs == nullptr or row_expert != nullptr): one wave per output column (weights streamed once
 // per row group); else the 64 x 64 MFMA tiles (offs: expert-grouped).
 constexpr int HY_GEMV_MAX_R = 8;
@@ -76,12 +79,18 @@ bool hy_linear_rows_is_gemv(const RowLinear& p);
 int hy_route_topk(const float* z, int ldz, int M, int top, int E, int32_t* row_expert, int32_t* row_tok, float* row_w,
                   int32_t* sort_tok, int32_t* sort_dst, float* sort_w, int32_t* offs, hipStream_t s);
 
-// Grouped softmax routing: scores = softmax(z[m, 0 : E]); the choice is made on score + correction[e] (correction
-// optional); the E experts form `groups` equal groups of neighbours, a group's score is its largest choice score, and
-// only experts of the `keep` best groups can be chosen; the `top` largest are taken (ties to the lower index
-// everywhere), weight = the chosen expert's score (not renormalised). Same outputs as hy_route_topk. E <= 1024,
-// E % groups == 0, groups <= 64, top <= keep * (E / groups).
-int hy_route_grouped(const float* z, int ldz, const float* correction, int M, int top, int E, int groups, int keep,
+// Grouped routing: scores = softmax(z[m, 0 : E]) or (sigmoid) sigmoid(z); the choice is made on score + correction[e]
+// (correction optional); the E experts form `groups` equal groups of neighbours, a group's score is the sum of its
+// `group_top` (1 or 2) largest choice scores, and only experts of the `keep` best groups can be chosen; the `top` largest
+// are taken (ties to the lower index everywhere), weight = w_scale * the chosen expert's score, with normalise also
+// divided by (the chosen scores' sum + 1e-20). Same outputs as hy_route_topk. E <= 1024, E % groups == 0, groups <= 64,
+// top <= keep * (E / groups).
+struct RouteRule {
+  int groups, keep, group_top;
+  int sigmoid, normalise;
+  float w_scale;
+};
+int hy_route_grouped(const float* z, int ldz, const float* correction, int M, int top, int E, RouteRule rule,
                      int32_t* row_expert, int32_t* row_tok, float* row_w, int32_t* sort_tok, int32_t* sort_dst,
                      float* sort_w, int32_t* offs, hipStream_t s);
 
@@ -118,6 +127,38 @@ int hy_norm_residual(const float* y, int nsum, float ysc, const float* w, int w_
 // products run on the packed GEMM, applied while the hidden activation is rounded for the second)
 typedef uint16_t bf16_t;
 int hy_cast_bf16(const float* x, bf16_t* y, long long n, int act, hipStream_t s);
+
+// out[m * ldo + c] = act(gu[m, c], gu[m, F + c]) for c < F: the gated epilogue of a product [M, 2F] that ran on the packed
+// GEMM; out fp32 or bf16, a column slice
+int hy_glu_rows(const float* gu, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
+                hipStream_t s);
+
+// h = tanh(alpha * x) * w + b, element by element (alpha one number, w and b [D]); h fp32 or bf16
+int hy_squash_rows(const float* x, int M, int D, const float* alpha, const float* w, const float* b, void* h, int h_bf16,
+                   hipStream_t s);
+
+// One residual step of a stack that averages over its depth. hist[j][M, D] (fp32) holds X_0 .. X_i:
+//   X = x + mult * (y [+ bias] [+ sum_{c < nsum} row_w[m * nsum + c] ye[m * nsum + c]]);  hist[i + 1] = X (if store);
+//   x_out = coef[i + 1] X + sum_{j <= i} coef[j] hist[j];  h = tanh(alpha x_out) w + b (with h: the next layer's input)
+struct DepthUpdate {
+  float* hist;
+  int M, D, i, store;
+  const float* x;  // [M, D]; x_out may be x
+  float* x_out;
+  float mult;
+  const float* y;     // [M, D]
+  const float* bias;  // optional [D]
+  const float* ye;    // optional [M * nsum, D], with row_w
+  int nsum;
+  const float* row_w;
+  const float* coef;  // [i + 2]
+  const float* alpha; // with h
+  const float* w;
+  const float* b;
+  void* h;            // optional [M, D] fp32 or bf16
+  int h_bf16;
+};
+int hy_depth_update(const DepthUpdate& p, hipStream_t s);
 
 // x <- cap * tanh(x / cap) in place (cap = 1: tanh), n elements
 int hy_softcap(float* x, long long n, float cap, hipStream_t s);
@@ -157,13 +198,15 @@ struct LatentPrep {
   void* cache;        // [B, 1, T, rank]
   int cbf16;
   float eps;
-  float* q;           // optional [M, q_cols]: dense copy of proj's columns [q_col0, q_col0 + q_cols) (the queries of the
-  int q_cols;         // same fused projection), for the linear that follows
+  void* q;            // optional [M, q_cols]: dense copy of proj's columns [q_col0, q_col0 + q_cols) (the queries of the
+  int q_cols;         // same fused projection), for the linear that follows; fp32, or (q_bf16) bf16
+  int q_bf16;
   int q_col0;
   const float* q_norm_w;  // optional [q_cols]: the copy is RMS-normed with this plain gain (a query latent)
   int row;                // width of a cache row, >= rank: the columns behind the latent, proj[col0 + rank, col0 + row), are
                           // cached as they are behind it, their first 2 rot_half numbers rotated by the token's position
-  const double* rot_freq; // optional [rot_half]: pair (2i, 2i + 1) turns by position * rot_freq[i]
+  const double* rot_freq; // optional [rot_half]: pair (2i, 2i + 1), or (rot_halves) (i, i + rot_half), turns by
+  int rot_halves;         // position * rot_freq[i]
   int rot_half;
   const int32_t* positions;  // [M], with rot_freq
 };
@@ -182,7 +225,9 @@ struct AttnBias {
   const float* bias;     // optional [nbias, H]: added to the score of distance n at row min(n, nbias - 1)
   int nbias;
   const float* sink;     // optional [H]: exp(sink[h]) joins the softmax denominator (no key, no value, not scaled)
-  float* out;  // [B * S, H * vdim]
+  void* out;   // [B * S, H * vdim] fp32, or (out_bf16) bf16; rows ldo apart
+  int ldo;
+  int out_bf16;
   int t_cap;   // keys the launch may have to cover (decode split sizing); <= T
   float* ws;   // decode split partials: B * H * splits * (vdim + 2) floats
   int splits;
@@ -191,8 +236,9 @@ struct AttnBias {
   const float* head_scale;  // optional [H]: head h's scores are (q . k * scale) * head_scale[h]
   int window;      // > 0 (chunk == 0): query at slot i sees key j <= i only if i - j < window or j < keep_first
   int keep_first;
-  const float* gate;  // optional: head h's output of token m is multiplied by sigmoid(gate[m * ldg + h])
-  int ldg;
+  const float* gate;  // optional: head h's output of token m is multiplied by sigmoid(gate[m * ldg + h]), or
+  int ldg;            // (gate_cols) its column c by sigmoid(gate[m * ldg + h * vdim + c])
+  int gate_cols;
   int ldv;         // elements between value rows (>= vdim; the values are the first vdim numbers of each row)
 };
 int hy_attn_bias(const AttnBias& p, hipStream_t s);
@@ -229,7 +275,8 @@ struct DeltaScan {
 int hy_delta_scan(const DeltaScan& p, hipStream_t s);
 
 // out[m * ldo + h * vdim + j] = x[m, h, j] / sqrt(mean_j(x^2) + eps) * w[w_heads ? h * vdim + j : j] *
-// act(gate[m * ldg + h * vdim + j]) * gain, act = silu (gate_act 0) or sigmoid (1). x = o, or with denom_floor [M, H]:
+// act(gate[m * ldg + h * vdim + j]) * gain, act = silu (gate_act 0), sigmoid (1) or no gate (2). x = o, or with
+// denom_floor [M, H]:
 // o is [M, H, vdim + 1] and x[m, h, j] = o[m, h, j] / (max(|o[m, h, vdim]|, denom_floor[m, h]) + 1e-6).
 struct GatedNorm {
   const float* o;
@@ -238,8 +285,9 @@ struct GatedNorm {
   const float* w;
   int w_heads;
   float eps;
-  float* out;
+  void* out;  // fp32, or (out_bf16) bf16
   int ldo;
+  int out_bf16;
   int M, H, vdim;
   int gate_act;
   const float* denom_floor;
@@ -267,6 +315,32 @@ struct RopePrep {
   int v_half;
 };
 int hy_rope_prep(const RopePrep& p, hipStream_t s);
+
+// The step after a fused q | k | v projection whose norms run over the whole q and the whole k: bias per column; q and k
+// divided by the root mean square of ALL their columns, times one gain per column; every q / k head rotated on its first
+// 2 half numbers, pairs (2i, 2i + 1) or (halves) (i, i + half), by position * freq[i]; values blended with another layer's
+// of the same token, v <- (1 - lambda) v + lambda v_prev; q to a dense buffer, k / v into the caches at slot + s.
+struct QkvPrep {
+  const float* proj;  // [M, ld]: q heads, k heads, v heads (more columns may follow)
+  int ld;
+  const float* bias;  // optional [H dim + G dim + G vdim]
+  const float* q_w;   // optional [H dim] (absent: no norm)
+  const float* k_w;   // optional [G dim]
+  float eps;
+  const int32_t* positions;  // [M]
+  const int32_t* slot;
+  int B, S, H, G, dim, vdim, T;
+  void* kc;  // [B, G, T, dim]
+  void* vc;  // [B, G, T, vdim]
+  int cbf16;
+  float* q;  // [M, H, dim]
+  const double* freq;  // [half]
+  int half, halves;
+  const float* v_prev;  // optional [M, G vdim], with lambda
+  const float* lambda;  // [1]
+  float* v_out;         // optional [M, G vdim]: the values as cached, in fp32
+};
+int hy_qkv_prep(const QkvPrep& p, hipStream_t s);
 
 // out[m * ldo + h * n + d] = gain * turn(a[m * lda + h * n + .], sign * positions[m])[d]: the first 2 half numbers of
 // every head rotated (freq == nullptr: none, a scaled copy)
@@ -296,6 +370,9 @@ int hy_mlstm_prep(const MlstmPrep& p, hipStream_t s);
 //       S <- keep S + write k [v, 1]^T;   o = S^T (q_scale q)
 //   mode 1 (a decay per key channel, bonus u for the current token, read before the write; cols = vdim):
 //       d = exp(-exp(decay + w0));   o = (S + diag(u) k v^T)^T q;   S <- diag(d) S + k v^T
+//   mode 2 (the forget gate decides what is written; read after the write; cols = vdim): k and q are pre-activations,
+//       i = u * sigmoid(-(k + w0)) (u: one minus the gate's lower bound, so the gate is 1 - i);
+//       S <- S + i (v^T - S);   o = S^T silu(q) q_scale
 struct LinScan {
   int mode;
   const float* q;  // token m, head h at q + m * ldq + h * dim
@@ -307,15 +384,15 @@ struct LinScan {
   const float* decay;  // mode 0: keep [M, H]; mode 1: pre-activations, token m, head h at decay + m * ldd + h * dim
   int ldd;
   const float* write;  // mode 0: [M, H]
-  const float* w0;     // mode 1: [H, dim]
-  const float* u;      // mode 1: [H, dim]
+  const float* w0;     // modes 1, 2: [H, dim]
+  const float* u;      // modes 1, 2: [H, dim]
   float* state;
   float* o;  // [M, H, cols]
   int B, S, H, dim, vdim;
   float q_scale;
   // nseg > 1: the sequence runs as nseg segments of seg_len tokens side by side (every segment non-empty), in three
   // launches (each segment's own final state and decay product, their combination, the scan proper from each segment's
-  // incoming state); seg_state holds B * nseg * H * dim * cols floats, seg_decay B * nseg * H (* dim in mode 1).
+  // incoming state); seg_state holds B * nseg * H * dim * cols floats, seg_decay B * nseg * H (* dim in modes 1, 2).
   // nseg == 1 (seg_len >= S): one launch.
   int nseg, seg_len;
   float* seg_state;

@@ -11,7 +11,8 @@
 //    walking the table; surplus workgroups exit), so one launch covers every expert of a token-sorted batch.
 //  * few rows (decode): a wave streams one or four weight rows once and dots them with up to 8 activation rows.
 //  * epilogues (RowAct): squared ReLU on one accumulator; gated forms accumulate the gate and the up rows of a column
-//    side by side: silu(g) * u, or the clamped form g' sigmoid(alpha g') (u' + 1) with g' = min(g, limit), u' = clamp(u).
+//    side by side: silu(g) * u, gelu_tanh(g) * u, or the clamped form g' sigmoid(alpha g') (u' + 1) with
+//    g' = min(g, limit), u' = clamp(u).
 //  * an optional per-row scale multiplies the activation row while it is staged (before the operand is rounded): the
 //    input-weighted experts of a score-routed mixture.
 // The table router's counting sort is here too.
@@ -107,6 +108,8 @@ JLA_DEV float lr_act(const RowLinear& p, float g, float u) {
     }
     case HY_ACT_SOFTCAP:
       return p.act_limit * tanhf(g / p.act_limit);
+    case HY_ACT_GELU_GLU:
+      return hy_gelu_tanh(g) * u;
     default:
       return g;
   }
@@ -351,7 +354,7 @@ bool hy_linear_rows_is_gemv(const RowLinear& p) {
 
 int hy_linear_rows(const RowLinear& p, hipStream_t s) {
   if (p.R < 0 || p.N <= 0 || p.K <= 0 || p.lda < p.K || p.ldo < p.N || p.E < 1) return -1;
-  if (p.act < HY_ACT_NONE || p.act > HY_ACT_SOFTCAP) return -8;
+  if (p.act < HY_ACT_NONE || p.act > HY_ACT_GELU_GLU) return -8;
   if (p.act == HY_ACT_SOFTCAP && !(p.act_limit > 0.f)) return -8;
   if (p.add_out && p.out_bf16) return -11;
   if (p.a_scale && p.a_bf16) return -9;  // (a bf16 copy cannot be scaled before its rounding)
@@ -549,9 +552,10 @@ __global__ void __launch_bounds__(256) route_topk_select_kernel(const float* z, 
 __global__ void route_sort_kernel(int R, int top, int E, const int32_t* row_expert, const float* row_w, int32_t* sort_tok,
                                   int32_t* sort_dst, float* sort_w, int32_t* offs);
 
-// Grouped softmax router, selection: one wave per token, logits in registers as above. Scores = softmax over all E
-// logits; choice = score + correction; a group's score is its largest choice; experts outside the `keep` best groups
-// are retired before the `top` rounds. The weight of a chosen expert is its score (without the correction).
+// Grouped router, selection: one wave per token, logits in registers as above. Scores = softmax over all E logits, or a
+// sigmoid of each; choice = score + correction; a group's score is its largest choice, or its two largest summed; experts
+// outside the `keep` best groups are retired before the `top` rounds. The weight of a chosen expert is its score (without
+// the correction), optionally over the chosen scores' sum, times a constant.
 JLA_DEV void rk_argmax(float& best, int& bi) {  // wave-wide (value, then lower index)
 #pragma unroll
   for (int off = 32; off; off >>= 1) {
@@ -565,9 +569,10 @@ JLA_DEV void rk_argmax(float& best, int& bi) {  // wave-wide (value, then lower 
 }
 
 __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* z, int ldz, const float* correction, int M,
-                                                                   int top, int E, int groups, int keep,
+                                                                   int top, int E, RouteRule rule,
                                                                    int32_t* row_expert, int32_t* row_tok, float* row_w) {
   const int lane = threadIdx.x & 63, m = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int groups = rule.groups, keep = rule.keep;
   if (m >= M) return;
   const float* zr = z + (size_t)m * ldz;
   float sc[RK_PER_LANE], ch[RK_PER_LANE];
@@ -583,10 +588,10 @@ __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* 
   float den = 0.f;
 #pragma unroll
   for (int u = 0; u < RK_PER_LANE; ++u) {
-    sc[u] = lane + 64 * u < E ? expf(sc[u] - zmax) : 0.f;
+    sc[u] = lane + 64 * u < E ? (rule.sigmoid ? hy_sigmoid(sc[u]) : expf(sc[u] - zmax)) : 0.f;
     den += sc[u];
   }
-  den = wave_sum(den);
+  den = rule.sigmoid ? 1.f : wave_sum(den);
 #pragma unroll
   for (int u = 0; u < RK_PER_LANE; ++u) {
     const int e = lane + 64 * u;
@@ -598,13 +603,24 @@ __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* 
     const int per = E / groups;
     float gs = -INFINITY;
     for (int g = 0; g < groups; ++g) {
-      float mx = -INFINITY;
+      float mx = -INFINITY, second = -INFINITY;
 #pragma unroll
       for (int u = 0; u < RK_PER_LANE; ++u) {
         const int e = lane + 64 * u;
-        if (e < E && e / per == g) mx = fmaxf(mx, ch[u]);
+        if (e < E && e / per == g) {
+          second = fmaxf(second, fminf(mx, ch[u]));
+          mx = fmaxf(mx, ch[u]);
+        }
       }
-      mx = wave_max(mx);
+      if (rule.group_top == 2 && per > 1) {
+        // the lane that holds the largest offers its own second largest, every other lane its largest
+        const float best = wave_max(mx);
+        const unsigned long long at = __ballot(mx == best);
+        const float rest = wave_max(lane == (int)__builtin_ctzll(at) ? second : mx);
+        mx = best + rest;
+      } else {
+        mx = wave_max(mx);
+      }
       if (lane == g) gs = mx;
     }
     unsigned long long kept = 0ull;
@@ -621,6 +637,7 @@ __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* 
     }
   }
   unsigned taken[RK_PER_LANE / 32 + 1] = {0};
+  float chosen = 0.f;
   for (int c = 0; c < top; ++c) {
     float best = -INFINITY, bw = 0.f;
     int bi = 0x7fffffff;
@@ -642,35 +659,49 @@ __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* 
         bw = best == -INFINITY ? 0.f : sc[u];
       }
     bw = wave_sum(bw);  // (one lane holds the chosen expert's score)
+    chosen += bw;
     if (lane == 0) {
       const int r = m * top + c;
       row_expert[r] = bi;
       row_tok[r] = m;
-      row_w[r] = bw;
+      row_w[r] = bw * rule.w_scale;
     }
   }
+  if (rule.normalise && lane == 0)  // (this lane wrote them)
+    for (int c = 0; c < top; ++c) row_w[m * top + c] /= chosen + 1e-20f;
 }
 
 // The same selection for at most 64 experts, one per lane, without serial rounds: a group's score by per-lane reads of
 // its members, then ranks (how many groups / experts come before this one, ties to the lower index) from reads of every
 // other lane, all independent of each other. A decode step's router is one token: its latency is what shows.
 __global__ void __launch_bounds__(256) route_grouped_select64_kernel(const float* z, int ldz, const float* correction,
-                                                                     int M, int top, int E, int groups, int keep,
+                                                                     int M, int top, int E, RouteRule rule,
                                                                      int32_t* row_expert, int32_t* row_tok, float* row_w) {
   const int lane = threadIdx.x & 63, m = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int groups = rule.groups, keep = rule.keep;
   if (m >= M) return;
   const bool valid = lane < E;
   float zv = valid ? z[(size_t)m * ldz + lane] : -INFINITY;
   const float cr = valid && correction ? correction[lane] : 0.f;
   zv = zv == zv ? zv : -INFINITY;
-  const float zmax = wave_max(zv);
-  const float ex = valid ? expf(zv - zmax) : 0.f;
-  const float sc = ex / wave_sum(ex);
+  float sc;
+  if (rule.sigmoid) {
+    sc = valid ? hy_sigmoid(zv) : 0.f;
+  } else {
+    const float zmax = wave_max(zv);
+    const float ex = valid ? expf(zv - zmax) : 0.f;
+    sc = ex / wave_sum(ex);
+  }
   float ch = valid ? sc + cr : -INFINITY;
   if (groups > 1) {
     const int per = E / groups, g = min(lane / per, groups - 1);
-    float gmax = -INFINITY;
-    for (int i = 0; i < per; ++i) gmax = fmaxf(gmax, __shfl(ch, g * per + i, 64));
+    float gmax = -INFINITY, gsec = -INFINITY;
+    for (int i = 0; i < per; ++i) {
+      const float o = __shfl(ch, g * per + i, 64);
+      gsec = fmaxf(gsec, fminf(gmax, o));
+      gmax = fmaxf(gmax, o);
+    }
+    if (rule.group_top == 2 && per > 1) gmax += gsec;
     int before = 0;  // groups ahead of this lane's
     for (int g2 = 0; g2 < groups; ++g2) {
       const float o = __shfl(gmax, g2 * per, 64);
@@ -683,26 +714,33 @@ __global__ void __launch_bounds__(256) route_grouped_select64_kernel(const float
     const float o = __shfl(ch, e2, 64);
     rank += (o > ch || (o == ch && e2 < lane)) ? 1 : 0;
   }
-  if (valid && rank < top) {
+  const bool take = valid && rank < top;
+  float wt = take && ch != -INFINITY ? sc : 0.f;
+  const float chosen = wave_sum(wt);
+  wt *= rule.w_scale;
+  if (rule.normalise) wt /= chosen + 1e-20f;
+  if (take) {
     const int r = m * top + rank;
     row_expert[r] = lane;
     row_tok[r] = m;
-    row_w[r] = ch == -INFINITY ? 0.f : sc;
+    row_w[r] = wt;
   }
 }
 
-int hy_route_grouped(const float* z, int ldz, const float* correction, int M, int top, int E, int groups, int keep,
+int hy_route_grouped(const float* z, int ldz, const float* correction, int M, int top, int E, RouteRule rule,
                      int32_t* row_expert, int32_t* row_tok, float* row_w, int32_t* sort_tok, int32_t* sort_dst,
                      float* sort_w, int32_t* offs, hipStream_t s) {
   if (M < 0 || top < 1 || E < 1 || E > RT_MAX_E || ldz < E) return -1;
+  const int groups = rule.groups, keep = rule.keep;
+  if (rule.group_top != 1 && rule.group_top != 2) return -4;
   if (groups < 1 || groups > 64 || E % groups || keep < 1 || keep > groups || top > keep * (E / groups)) return -3;
   if (M == 0) return 0;
   if (E <= 64)
-    route_grouped_select64_kernel<<<(M + 3) / 4, 256, 0, s>>>(z, ldz, correction, M, top, E, groups, keep, row_expert,
-                                                              row_tok, row_w);
+    route_grouped_select64_kernel<<<(M + 3) / 4, 256, 0, s>>>(z, ldz, correction, M, top, E, rule, row_expert, row_tok,
+                                                              row_w);
   else
-    route_grouped_select_kernel<<<(M + 3) / 4, 256, 0, s>>>(z, ldz, correction, M, top, E, groups, keep, row_expert,
-                                                            row_tok, row_w);
+    route_grouped_select_kernel<<<(M + 3) / 4, 256, 0, s>>>(z, ldz, correction, M, top, E, rule, row_expert, row_tok,
+                                                            row_w);
   JLA_CHECK_LAUNCH();
   if (!sort_tok) return 0;
   if (!sort_dst || !sort_w || !offs) return -2;

@@ -1,7 +1,9 @@
 // Row kernels of the hybrid stack: embedding-slice gather, the norm on a sublayer's OUTPUT fused with the residual add
 // (x += rms_norm(sum of the chosen experts' outputs) * w, w one number or a vector), the per-layer token-side gate
 // (gelu_tanh(gate projection) * a slice of a second embedding table), the latent-attention prep (normed latent, normed
-// query latent, rotated shared key part, cache write) and the hyper-connection update of several residual streams.
+// query latent, rotated shared key part, cache write), the hyper-connection update of several residual streams, and the
+// residual step of a depth-averaging stack (residual add, weighted sum of every earlier layer's result, the next layer's
+// statistics-free norm: everything is element by element, so one pass serves all three).
 // fp32 statistics and residual.
 #include "hy_util.h"
 #include "hybrid.h"
@@ -162,10 +164,6 @@ int hy_softcap(float* x, long long n, float cap, hipStream_t s) {
   return 0;
 }
 
-JLA_DEV float ns_gelu_tanh(float z) {
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
-
 template <typename WT>
 __global__ void __launch_bounds__(256) gelu_gate_rows_kernel(const float* gp, const int32_t* ids, const WT* table, int V,
                                                              int ld, int col0, float* g, int D) {
@@ -173,7 +171,7 @@ __global__ void __launch_bounds__(256) gelu_gate_rows_kernel(const float* gp, co
   int id = ids[m];
   id = id < 0 || id >= V ? 0 : id;
   const WT* row = table + (size_t)id * ld + col0;
-  for (int d = threadIdx.x; d < D; d += 256) g[(size_t)m * D + d] = ns_gelu_tanh(gp[(size_t)m * D + d]) * ns_ld(row + d);
+  for (int d = threadIdx.x; d < D; d += 256) g[(size_t)m * D + d] = hy_gelu_tanh(gp[(size_t)m * D + d]) * ns_ld(row + d);
 }
 
 int hy_gelu_gate_rows(const float* gp, const int32_t* ids, const void* table, int wbf16, int V, int ld, int col0,
@@ -206,7 +204,11 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep p) {
   const int tid = threadIdx.x, m = blockIdx.x;
   if (p.q) {
     const float* src = p.proj + (size_t)m * p.ld + p.q_col0;
-    float* dst = p.q + (size_t)m * p.q_cols;
+    auto put = [&](int d, float v) {
+      const size_t at = (size_t)m * p.q_cols + d;
+      if (p.q_bf16) reinterpret_cast<bf16_t*>(p.q)[at] = f2bf(v);
+      else reinterpret_cast<float*>(p.q)[at] = v;
+    };
     float qsc = 1.f;
     if (p.q_norm_w) {  // a query latent: RMS over the copied columns
       float qs = 0.f;
@@ -231,7 +233,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep p) {
       }
 #pragma unroll
       for (int u = 0; u < 4; ++u)
-        if (d0 + tid + 256 * u < p.q_cols) dst[d0 + tid + 256 * u] = p.q_norm_w ? v[u] * qsc * g[u] : v[u];
+        if (d0 + tid + 256 * u < p.q_cols) put(d0 + tid + 256 * u, p.q_norm_w ? v[u] * qsc * g[u] : v[u]);
     }
   }
   const float* row = p.proj + (size_t)m * p.ld + p.col0;
@@ -256,7 +258,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep p) {
   const int b = m / p.S, t = *p.slot + (m - b * p.S);
   if (t < 0 || t >= p.T) return;  // cache full: the write is dropped
   CT* dst = reinterpret_cast<CT*>(p.cache) + ((size_t)b * p.T + t) * p.row;
-  // behind the latent: the shared key part, rotated in pairs (2i, 2i + 1) by the token's position
+  // behind the latent: the shared key part, rotated in pairs (2i, 2i + 1) or (i, i + half) by the token's position
   const int tail = p.row - p.rank;
   if (tail > 0) {
     const float* tr = row + p.rank;
@@ -264,9 +266,10 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep p) {
     for (int i = tid; i < p.rot_half; i += 256) {
       float sn, cs;
       lp_sincos(pos, p.rot_freq[i], &sn, &cs);
-      const float a = tr[2 * i], c = tr[2 * i + 1];
-      lp_st(dst + p.rank + 2 * i, a * cs - c * sn);
-      lp_st(dst + p.rank + 2 * i + 1, c * cs + a * sn);
+      const int ia = p.rot_halves ? i : 2 * i, ic = p.rot_halves ? i + p.rot_half : 2 * i + 1;
+      const float a = tr[ia], c = tr[ic];
+      lp_st(dst + p.rank + ia, a * cs - c * sn);
+      lp_st(dst + p.rank + ic, c * cs + a * sn);
     }
     for (int d = 2 * p.rot_half + tid; d < tail; d += 256) lp_st(dst + p.rank + d, tr[d]);
   }
@@ -388,6 +391,185 @@ int hy_hc_update(const HyperUpdate& p, hipStream_t s) {
     HC_WIDE(9); HC_WIDE(10); HC_WIDE(11); HC_WIDE(12); HC_WIDE(13); HC_WIDE(14); HC_WIDE(15); HC_WIDE(16);
 #undef HC_WIDE
   }
+  JLA_CHECK_LAUNCH();
+  return 0;
+}
+
+// ---- depth average -------------------------------------------------------------------------------------------------
+// V consecutive columns of one token per thread (V = 4: 16-byte accesses, D a multiple of 4). Loads of the sublayers'
+// results and of the earlier planes do not depend on each other and go out together.
+template <int V>
+JLA_DEV void dv_load(const float* p, float* f) {
+  if constexpr (V == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(p);
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+  } else {
+    f[0] = *p;
+  }
+}
+template <int V>
+JLA_DEV void dv_store(float* p, const float* f) {
+  if constexpr (V == 4) *reinterpret_cast<float4*>(p) = float4{f[0], f[1], f[2], f[3]};
+  else *p = f[0];
+}
+template <int V>
+JLA_DEV void dv_store_h(void* h, int bf, size_t at, const float* f) {
+  if (!bf) {
+    dv_store<V>(reinterpret_cast<float*>(h) + at, f);
+  } else if constexpr (V == 4) {
+    *reinterpret_cast<uint2*>(reinterpret_cast<bf16_t*>(h) + at) =
+        uint2{(uint32_t)f2bf(f[0]) | (uint32_t)f2bf(f[1]) << 16, (uint32_t)f2bf(f[2]) | (uint32_t)f2bf(f[3]) << 16};
+  } else {
+    reinterpret_cast<bf16_t*>(h)[at] = f2bf(f[0]);
+  }
+}
+
+template <int V>
+__global__ void __launch_bounds__(256) depth_update_kernel(DepthUpdate p, long long n) {
+  const long long t = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= n) return;
+  const int dv = p.D / V;
+  const int m = (int)(t / dv), c = (int)(t - (long long)m * dv) * V;
+  const size_t at = (size_t)m * p.D + c, plane = (size_t)p.M * p.D;
+  float x[V], y[V], acc[V];
+  dv_load<V>(p.x + at, x);
+  dv_load<V>(p.y + at, y);
+  if (p.bias) {
+    float bv[V];
+    dv_load<V>(p.bias + c, bv);
+#pragma unroll
+    for (int k = 0; k < V; ++k) y[k] += bv[k];
+  }
+  if (p.ye) {
+    const float* ye = p.ye + (size_t)m * p.nsum * p.D + c;
+    const float* rw = p.row_w + (size_t)m * p.nsum;
+#pragma unroll 4
+    for (int q = 0; q < p.nsum; ++q) {
+      float yv[V];
+      dv_load<V>(ye + (size_t)q * p.D, yv);
+      const float w = rw[q];
+#pragma unroll
+      for (int k = 0; k < V; ++k) y[k] = fmaf(w, yv[k], y[k]);
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < V; ++k) acc[k] = 0.f;
+#pragma unroll 8
+  for (int j = 0; j <= p.i; ++j) {
+    float hv[V];
+    dv_load<V>(p.hist + j * plane + at, hv);
+    const float cf = p.coef[j];
+#pragma unroll
+    for (int k = 0; k < V; ++k) acc[k] = fmaf(cf, hv[k], acc[k]);
+  }
+  const float cn = p.coef[p.i + 1];
+#pragma unroll
+  for (int k = 0; k < V; ++k) {
+    x[k] = fmaf(p.mult, y[k], x[k]);
+    acc[k] = fmaf(cn, x[k], acc[k]);
+  }
+  if (p.store) dv_store<V>(p.hist + (p.i + 1) * plane + at, x);
+  dv_store<V>(p.x_out + at, acc);
+  if (p.h) {
+    const float al = *p.alpha;
+    float wv[V], bv[V];
+    dv_load<V>(p.w + c, wv);
+    dv_load<V>(p.b + c, bv);
+#pragma unroll
+    for (int k = 0; k < V; ++k) acc[k] = fmaf(tanhf(al * acc[k]), wv[k], bv[k]);
+    dv_store_h<V>(p.h, p.h_bf16, at, acc);
+  }
+}
+
+// small steps (a few tokens) as one-wave workgroups, so that they spread over more compute units
+static int dv_threads(long long n) { return n <= 64LL * 512 ? 64 : 256; }
+
+int hy_depth_update(const DepthUpdate& p, hipStream_t s) {
+  if (p.M < 0 || p.D < 1 || p.i < 0 || !p.hist || !p.x || !p.x_out || !p.y || !p.coef) return -1;
+  if (p.ye && (!p.row_w || p.nsum < 1)) return -2;
+  if (p.h && (!p.alpha || !p.w || !p.b)) return -3;
+  if (p.M == 0) return 0;
+  const int v = p.D % 4 == 0 ? 4 : 1;
+  const long long n = (long long)p.M * (p.D / v);
+  const int th = dv_threads(n);
+  if ((n + th - 1) / th > 0x7fffffffLL) return -4;
+  if (v == 4) depth_update_kernel<4><<<(unsigned)((n + th - 1) / th), th, 0, s>>>(p, n);
+  else depth_update_kernel<1><<<(unsigned)((n + th - 1) / th), th, 0, s>>>(p, n);
+  JLA_CHECK_LAUNCH();
+  return 0;
+}
+
+template <int V>
+__global__ void __launch_bounds__(256) squash_rows_kernel(const float* __restrict__ x, int D, const float* alpha,
+                                                          const float* w, const float* b, void* h, int h_bf16,
+                                                          long long n) {
+  const long long t = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= n) return;
+  const int dv = D / V;
+  const long long m = t / dv;
+  const int c = (int)(t - m * dv) * V;
+  const size_t at = (size_t)m * D + c;
+  float f[V], wv[V], bv[V];
+  dv_load<V>(x + at, f);
+  dv_load<V>(w + c, wv);
+  dv_load<V>(b + c, bv);
+  const float al = *alpha;
+#pragma unroll
+  for (int k = 0; k < V; ++k) f[k] = fmaf(tanhf(al * f[k]), wv[k], bv[k]);
+  dv_store_h<V>(h, h_bf16, at, f);
+}
+
+int hy_squash_rows(const float* x, int M, int D, const float* alpha, const float* w, const float* b, void* h, int h_bf16,
+                   hipStream_t s) {
+  if (M < 0 || D < 1 || !x || !alpha || !w || !b || !h) return -1;
+  if (M == 0) return 0;
+  const int v = D % 4 == 0 ? 4 : 1;
+  const long long n = (long long)M * (D / v);
+  const int th = dv_threads(n);
+  if ((n + th - 1) / th > 0x7fffffffLL) return -2;
+  if (v == 4) squash_rows_kernel<4><<<(unsigned)((n + th - 1) / th), th, 0, s>>>(x, D, alpha, w, b, h, h_bf16, n);
+  else squash_rows_kernel<1><<<(unsigned)((n + th - 1) / th), th, 0, s>>>(x, D, alpha, w, b, h, h_bf16, n);
+  JLA_CHECK_LAUNCH();
+  return 0;
+}
+
+// V columns of one token per thread: the gated activation of a product whose gate and up columns lie side by side
+template <int V>
+__global__ void __launch_bounds__(256) glu_rows_kernel(const float* __restrict__ gu, int F, int act, float limit,
+                                                       float alpha, void* out, int out_bf16, int ldo, long long n) {
+  const long long t = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (t >= n) return;
+  const int fv = F / V;
+  const long long m = t / fv;
+  const int c = (int)(t - m * fv) * V;
+  float g[V], u[V];
+  dv_load<V>(gu + (size_t)m * 2 * F + c, g);
+  dv_load<V>(gu + (size_t)m * 2 * F + F + c, u);
+#pragma unroll
+  for (int k = 0; k < V; ++k) {
+    if (act == HY_ACT_SWIGLU) {
+      g[k] = hy_silu(g[k]) * u[k];
+    } else if (act == HY_ACT_GELU_GLU) {
+      g[k] = hy_gelu_tanh(g[k]) * u[k];
+    } else {
+      const float gc = fminf(g[k], limit), uc = fminf(fmaxf(u[k], -limit), limit);
+      g[k] = gc * hy_sigmoid(alpha * gc) * (uc + 1.f);
+    }
+  }
+  dv_store_h<V>(out, out_bf16, (size_t)m * ldo + c, g);
+}
+
+int hy_glu_rows(const float* gu, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
+                hipStream_t s) {
+  if (M < 0 || F < 1 || ldo < F || !hy_act_gated(act)) return -1;
+  if (M == 0) return 0;
+  const uintptr_t mask = out_bf16 ? 7 : 15;
+  const int v = F % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out & mask) == 0 ? 4 : 1;
+  const long long n = (long long)M * (F / v);
+  if ((n + 255) / 256 > 0x7fffffffLL) return -2;
+  const unsigned grid = (unsigned)((n + 255) / 256);
+  if (v == 4) glu_rows_kernel<4><<<grid, 256, 0, s>>>(gu, F, act, limit, alpha, out, out_bf16, ldo, n);
+  else glu_rows_kernel<1><<<grid, 256, 0, s>>>(gu, F, act, limit, alpha, out, out_bf16, ldo, n);
   JLA_CHECK_LAUNCH();
   return 0;
 }

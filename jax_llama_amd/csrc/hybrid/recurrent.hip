@@ -9,11 +9,13 @@
 //                    values as wave-uniform scalars.
 //   hy_lin_scan    : S <- D_t S + b_t k_t v_t^T with the read-out after the write (scalar D, b: the exponential-gate
 //                    memory; its normaliser is one more value column whose value is 1) or before it with a bonus for the
-//                    current token (per-channel D from a double exponential: the time-mix memory). Thread layout of the
+//                    current token (per-channel D from a double exponential: the time-mix memory), or with the write
+//                    factor one minus the per-channel keep factor and no key (a gated running average of the values:
+//                    S <- S + i (v^T - S), read after the write). Thread layout of the
 //                    delta-rule scan: a thread owns 16 key rows of one state column in registers, the lanes of a column
 //                    combine their partial read-outs by lane exchange, tokens are staged through LDS a chunk at a time
 //                    with the next chunk's loads in flight. A long sequence is cut into segments that run side by side
-//                    (both recurrences are linear in the state): segment states and decay products, one combining
+//                    (every recurrence is linear in the state): segment states and decay products, one combining
 //                    walk, then the scan proper from every segment's incoming state.
 #include "hy_util.h"
 #include "hybrid.h"
@@ -108,7 +110,8 @@ constexpr int LS_PITCH = 20;    // floats between the staged slices: the lanes' 
 constexpr int LS_STAGE = 4096;  // floats of one staged chunk of tokens in LDS
 constexpr int LS_PF = LS_STAGE / 256;
 
-// Staged element i of the chunk starting at token s0. Per token: [k (dimp) | q (dimp) | MODE 1: decay (dimp) |
+// Staged element i of the chunk starting at token s0. Per token: [k (MODE 2: the write gate) (dimp) | q (dimp) |
+// MODE 1: decay (dimp) |
 // v (cols) | MODE 0: keep, write | pad]; dimp = R slices of LS_PITCH floats (16 values + 4 pad; zeros past dim), cols =
 // the block's state columns [j0, j0 + cols).
 // Staging is split in three so that a thread's 16 loads of a chunk are all in flight together and cost a few
@@ -136,7 +139,7 @@ JLA_DEV LsPlan ls_plan(const LinScan& p, int h, int j0, int cols, int dimp, int 
   const int c = e - NV * dimp, j = j0 + c;
   const bool is_v = !vec && c < cols, is_g = MODE == 0 && !vec && (c == cols || c == cols + 1);
   const int src = vec ? which : is_v ? LS_SRC_V : is_g ? (c == cols ? LS_SRC_KEEP : LS_SRC_WRITE) : LS_SRC_K;
-  const int code = vec ? (pad ? LS_ZERO : which == 1 ? LS_QUERY : which == 2 ? LS_DECAY : LS_PLAIN)
+  const int code = vec ? (pad ? LS_ZERO : which == 1 ? LS_QUERY : which == (MODE == 2 ? 0 : 2) ? LS_DECAY : LS_PLAIN)
                        : is_v ? ((MODE == 0 && j >= p.vdim) ? LS_ONE : LS_PLAIN)  // (the normaliser's column: value 1)
                               : is_g ? LS_PLAIN : LS_ZERO;
   LsPlan r;
@@ -146,8 +149,11 @@ JLA_DEV LsPlan ls_plan(const LinScan& p, int h, int j0, int cols, int dimp, int 
 }
 
 template <int MODE>
-JLA_DEV float ls_val(int code, float raw, float w0v, float q_scale) {
+JLA_DEV float ls_val(int code, float raw, float w0v, float uv, float q_scale) {
   if (MODE == 1 && code == LS_DECAY) return expf(-expf(raw + w0v));
+  // one minus the forget gate, taken directly: a gate near 1 keeps the write factor's full accuracy
+  if (MODE == 2 && code == LS_DECAY) return uv * hy_sigmoid(-(raw + w0v));
+  if (MODE == 2 && code == LS_QUERY) return hy_silu(raw) * q_scale;
   return code == LS_ZERO ? 0.f : code == LS_ONE ? 1.f : code == LS_QUERY ? raw * q_scale : raw;
 }
 
@@ -192,23 +198,24 @@ __global__ void __launch_bounds__(256) lin_scan_kernel(LinScan p, const float* s
   constexpr int cols = 256 / R, dimp = R * LS_PITCH;
   const int j0 = blockIdx.x * cols, jl = j - j0;
   constexpr int NV = MODE == 1 ? 3 : 2;
-  float S[LS_SLICE], uu[LS_SLICE], dprod[MODE == 1 ? LS_SLICE : 1];
+  float S[LS_SLICE], uu[LS_SLICE], dprod[MODE != 0 ? LS_SLICE : 1];
   const size_t sidx = ((((size_t)b * p.nseg + seg) * p.H + h) * p.dim) * ncols + jc;  // (b, segment, head) of a state array
 #pragma unroll
   for (int i = 0; i < LS_SLICE; ++i) {
     const bool in = i0 + i < p.dim;
     S[i] = (s_init && live && in) ? s_init[sidx + (size_t)(i0 + i) * ncols] : 0.f;
     uu[i] = (MODE == 1 && in) ? p.u[(size_t)h * p.dim + i0 + i] : 0.f;
-    if (MODE == 1) dprod[i] = 1.f;
+    if (MODE != 0) dprod[i] = 1.f;
   }
   if (MODE == 0) dprod[0] = 1.f;
-  float pf[LS_PF], pw[LS_PF];
+  float pf[LS_PF], pw[LS_PF], pu[MODE == 2 ? LS_PF : 1];
   LsPlan plan[LS_PF];
 #pragma unroll
   for (int u = 0; u < LS_PF; ++u) {
     plan[u] = ls_plan<MODE>(p, h, j0, cols, dimp, per, per_magic, tid + 256 * u);
     // (the decay's offset does not depend on the token: loaded once)
-    pw[u] = (MODE == 1 && (plan[u].meta & 7) == LS_DECAY) ? p.w0[plan[u].off] : 0.f;
+    pw[u] = (MODE != 0 && (plan[u].meta & 7) == LS_DECAY) ? p.w0[plan[u].off] : 0.f;
+    if (MODE == 2) pu[u] = (plan[u].meta & 7) == LS_DECAY ? p.u[plan[u].off] : 0.f;
   }
   const size_t row0 = (size_t)b * p.S;
   // loads of the chunk at token sn (n floats of it): every thread issues all of its loads before any is used
@@ -228,7 +235,7 @@ __global__ void __launch_bounds__(256) lin_scan_kernel(LinScan p, const float* s
 #pragma unroll
     for (int u = 0; u < LS_PF; ++u) {
       const int i = tid + 256 * u;
-      if (i < n) stage[i] = ls_val<MODE>(plan[u].meta & 7, pf[u], pw[u], p.q_scale);
+      if (i < n) stage[i] = ls_val<MODE>(plan[u].meta & 7, pf[u], pw[u], pu[MODE == 2 ? u : 0], p.q_scale);
     }
   };
   fetch(t_lo, min(ct, t_hi - t_lo) * per);
@@ -260,6 +267,20 @@ __global__ void __launch_bounds__(256) lin_scan_kernel(LinScan p, const float* s
         for (int i = 0; i < LS_SLICE; i += 2) {
           S[i] = fmaf(keep, S[i], kv[i] * wv);
           S[i + 1] = fmaf(keep, S[i + 1], kv[i + 1] * wv);
+          if (!STATE_ONLY) {
+            o0 = fmaf(S[i], qv[i], o0);
+            o1 = fmaf(S[i + 1], qv[i + 1], o1);
+          }
+        }
+      } else if (MODE == 2) {
+#pragma unroll
+        for (int i = 0; i < LS_SLICE; i += 2) {
+          if (STATE_ONLY) {
+            dprod[i] *= 1.f - kv[i];
+            dprod[i + 1] *= 1.f - kv[i + 1];
+          }
+          S[i] = fmaf(kv[i], v - S[i], S[i]);
+          S[i + 1] = fmaf(kv[i + 1], v - S[i + 1], S[i + 1]);
           if (!STATE_ONLY) {
             o0 = fmaf(S[i], qv[i], o0);
             o1 = fmaf(S[i + 1], qv[i + 1], o1);
@@ -311,7 +332,7 @@ __global__ void __launch_bounds__(256) lin_scan_kernel(LinScan p, const float* s
     } else {
 #pragma unroll
       for (int i = 0; i < LS_SLICE; ++i)
-        if (i0 + i < p.dim) seg_decay[d0 * p.dim + i0 + i] = dprod[MODE == 1 ? i : 0];
+        if (i0 + i < p.dim) seg_decay[d0 * p.dim + i0 + i] = dprod[MODE != 0 ? i : 0];
     }
   }
 }
@@ -337,11 +358,12 @@ __global__ void __launch_bounds__(256) lin_combine_kernel(float* state, float* s
 }
 
 int hy_lin_scan(const LinScan& p, hipStream_t s) {
-  if (p.mode != 0 && p.mode != 1) return -1;
+  if (p.mode < 0 || p.mode > 2) return -1;
   if (p.B < 0 || p.S < 1 || p.H < 1 || p.dim < 1 || p.vdim < 1) return -1;
   if (p.dim > 64 * LS_SLICE) return -2;
   if (p.ldq < p.H * p.dim || p.ldk < p.H * p.dim || p.ldv < p.H * p.vdim) return -5;
-  if (p.mode == 1 && (p.ldd < p.H * p.dim || !p.w0 || !p.u)) return -6;
+  if (p.mode == 1 && p.ldd < p.H * p.dim) return -6;
+  if (p.mode != 0 && (!p.w0 || !p.u)) return -6;
   if (p.mode == 0 && !p.write) return -6;
   if (p.B == 0) return 0;
   if (p.H > 65535 || p.B > 65535) return -3;
@@ -361,12 +383,15 @@ int hy_lin_scan(const LinScan& p, hipStream_t s) {
     static_assert(ls_per(1, RR) <= LS_STAGE, "a staged token fits");                                             \
     if (!cut) {                                                                                                  \
       if (p.mode == 0) lin_scan_kernel<0, RR, 0><<<grid, 256, 0, s>>>(p, p.state, p.state, nullptr);             \
+      else if (p.mode == 2) lin_scan_kernel<2, RR, 0><<<grid, 256, 0, s>>>(p, p.state, p.state, nullptr);        \
       else lin_scan_kernel<1, RR, 0><<<grid, 256, 0, s>>>(p, p.state, p.state, nullptr);                         \
     } else if (pass == 0) {                                                                                      \
       if (p.mode == 0) lin_scan_kernel<0, RR, 1><<<grid, 256, 0, s>>>(p, nullptr, p.seg_state, p.seg_decay);     \
+      else if (p.mode == 2) lin_scan_kernel<2, RR, 1><<<grid, 256, 0, s>>>(p, nullptr, p.seg_state, p.seg_decay); \
       else lin_scan_kernel<1, RR, 1><<<grid, 256, 0, s>>>(p, nullptr, p.seg_state, p.seg_decay);                 \
     } else {                                                                                                     \
       if (p.mode == 0) lin_scan_kernel<0, RR, 0><<<grid, 256, 0, s>>>(p, p.seg_state, nullptr, nullptr);         \
+      else if (p.mode == 2) lin_scan_kernel<2, RR, 0><<<grid, 256, 0, s>>>(p, p.seg_state, nullptr, nullptr);    \
       else lin_scan_kernel<1, RR, 0><<<grid, 256, 0, s>>>(p, p.seg_state, nullptr, nullptr);                     \
     }                                                                                                            \
     break
@@ -386,7 +411,7 @@ int hy_lin_scan(const LinScan& p, hipStream_t s) {
     if (cut && pass == 0) {
       const long long n = (long long)p.B * p.H * p.dim * ncols;
       lin_combine_kernel<<<(unsigned)((n + 255) / 256), 256, 0, s>>>(p.state, p.seg_state, p.seg_decay, p.nseg, p.H, p.dim,
-                                                                    ncols, p.mode == 1, n);
+                                                                    ncols, p.mode != 0, n);
       JLA_CHECK_LAUNCH();
     }
   }

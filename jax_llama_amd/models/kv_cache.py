@@ -110,6 +110,7 @@ class HybridCache:
         ``[B, H, dim, vdim + 1]`` and the running maximum of its gates ``[B, H]`` (fp32);
       * ``("timemix", heads, dim, vdim, width)``: a matrix memory ``[B, H, dim, vdim]`` and the previous token's
         mixer input ``[B, width]`` (fp32);
+      * ``("linear", heads, dim, vdim)``: a matrix state alone ``[B, H, dim, vdim]`` (fp32);
       * ``("multi", spec, spec, ...)``: a layer whose mixers run side by side, each with its own entry (at most one
         that holds keys and one that is recurrent);
       * ``None``: nothing.
@@ -139,7 +140,7 @@ class HybridCache:
         if sp[0] == "multi":
             kinds = [p[0] for p in sp[1:]]
             if sum(k in ("kv", "latent", "kv_from") for k in kinds) > 1 or \
-                    sum(k in ("delta", "mlstm", "timemix") for k in kinds) > 1:
+                    sum(k in ("delta", "mlstm", "timemix", "linear") for k in kinds) > 1:
                 raise ValueError(f"a layer holds at most one key / value entry and one recurrent entry: {sp!r}")
             return list(sp[1:])
         return [sp]
@@ -168,6 +169,8 @@ class HybridCache:
             _, h, dim, vdim, width = sp
             self._state[i] = torch.zeros(batch_size, h, dim, vdim, **f32)
             self._conv[i] = torch.zeros(batch_size, width, **f32)
+        elif sp[0] == "linear":
+            self._state[i] = torch.zeros(batch_size, *sp[1:], **f32)
         else:
             raise ValueError(f"unknown cache spec {sp!r}")
 
@@ -188,8 +191,9 @@ class HybridCache:
 
     def recurrent(self, i: int):
         """The two carried tensors of a recurrent layer: ``(state, convolution tail)`` (delta), ``(state with the
-        normaliser column, running maximum)`` (mlstm) or ``(state, previous token's input)`` (timemix)."""
-        return self._state[i], self._conv[i]
+        normaliser column, running maximum)`` (mlstm), ``(state, previous token's input)`` (timemix) or ``(state, None)``
+        (linear)."""
+        return self._state[i], self._conv.get(i)
 
     def advance(self, n: int) -> None:
         self.index += n
@@ -233,6 +237,8 @@ class HybridCache:
                     n += 4 * batch_size * sp[1] * (sp[2] * (sp[3] + 1) + 1)
                 elif sp[0] == "timemix":
                     n += 4 * batch_size * (sp[1] * sp[2] * sp[3] + sp[4])
+                elif sp[0] == "linear":
+                    n += 4 * batch_size * sp[1] * sp[2] * sp[3]
         return n
 
 
@@ -267,4 +273,4 @@ class HybridCacheRows:
 
     def recurrent(self, i: int):
         s, c = self.parent.recurrent(i)
-        return s[self.b0:self.b1], c[self.b0:self.b1]
+        return s[self.b0:self.b1], c[self.b0:self.b1] if c is not None else None

@@ -45,8 +45,9 @@ class LayerListLM:
         self.embed_scale = 1.0
         self.embed_norm: Optional[torch.Tensor] = None  # fp32 [D]: gain of an RMS norm on the embedding
         self.logit_softcap = 0.0                        # logits <- cap * tanh(logits / cap) when > 0
+        self.depth_history = False  # the blocks average over all layers' results (mixers.DepthAverageBlock)
         self.streams = 0  # > 0: the blocks work on that many residual streams [S, M, D] (hyper-connections)
-        self.final_norm: Optional[torch.Tensor] = None  # fp32 gain of the last norm: one number or [D]
+        self.final_norm = None  # gain of the last RMS norm (fp32, one number or [D]), or an hy.SquashNorm
         self.head: Optional[torch.Tensor] = None
         if _do_init:
             self.load_state_dict(self.random_state_dict(config, seed))
@@ -137,6 +138,20 @@ class LayerListLM:
                 if collect_hidden:
                     hidden.append(hy.hc_in(xs, ones).reshape(b, s, d))
             x = ctx.u if ctx.u is not None else hy.hc_in(xs, ones)
+        elif self.depth_history:
+            # plane 0 holds the embedding, a block adds its result, writes what goes on to x and leaves the next layer's
+            # normed input in ctx.h
+            ctx.hist = torch.empty(len(self.blocks) + 1, b * s, d, dtype=F32, device=self.device)
+            x = hy.embed_rows(idf, self.embed, scale=self.embed_scale, out=ctx.hist[0])
+            ctx.act_dtype = BF16 if hy.prompt_bf16(b * s, d, self.param_dtype) else F32
+            ctx.every_row = logits_mode == "all" or (s == 1 and logits_mode in ("last", "argmax"))
+            if self.blocks:
+                ctx.h = hy.squash_rows(x, self.blocks[0].norm, ctx.act_dtype)
+                x = torch.empty_like(x)
+            for blk in self.blocks:
+                blk(x, ctx)
+                if collect_hidden:
+                    hidden.append(x.reshape(b, s, d).clone())
         else:
             x = hy.embed_rows(idf, self.embed, scale=self.embed_scale)
             if self.embed_norm is not None:
@@ -156,7 +171,11 @@ class LayerListLM:
         else:
             raise ValueError(f"unknown logits_mode {logits_mode!r}")
         cap = float(self.logit_softcap or 0.0)
-        logits = hy.linear(hy.rms_rows(xl, self.final_norm, self.eps), self.head,
+        if isinstance(self.final_norm, hy.SquashNorm):
+            xf = ctx.h if ctx.every_row and ctx.h is not None else hy.squash_rows(xl, self.final_norm)
+        else:
+            xf = hy.rms_rows(xl, self.final_norm, self.eps)
+        logits = hy.linear(xf, self.head,
                            act=hy.ACT_SOFTCAP if cap > 0 else hy.ACT_NONE, limit=cap)
         return logits, x, hidden, []
 

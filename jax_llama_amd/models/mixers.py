@@ -33,7 +33,19 @@ the same mechanisms with other values.
   HyperBlock      : pre-norm sublayers over several residual streams (hyper-connections): a sublayer reads a weighted
                     sum of the streams, and its result is added to a mixed copy of them.
 
-The blocks of the group before the last split a sublayer into ``features(h, ctx, out=None, gain=1.0)`` (everything up to the output
+  WholeNormAttention : projection biases, RMS norms over the whole q and k projections, interleaved rotary positions, a
+                    sliding window, a constant one in the softmax denominator, values blended with the first such layer's,
+                    a sigmoid gate per output column.
+  GatedRunningMixer : linear attention whose forget gate also decides what is written (a gated running average of the
+                    values per key channel), no key of its own.
+  GatedMoE        : gated (two-accumulator) experts chosen by a grouped router, weights on their output, shared expert.
+  DepthAverageBlock : mixer and feed-forward side by side on one statistics-free norm; the layer's result joins a history
+                    of all layers' results, and the next layer reads a weighted sum of them.
+
+The mixers of the last group split into ``features(proj, ctx, out)`` -- everything between the fused input projection
+``w_in`` and the output matrix ``w_o`` -- so that their block can fuse other rows (a router) into the input product and run
+one output product over the features of all of its members.
+The blocks of the group before the last two split a sublayer into ``features(h, ctx, out=None, gain=1.0)`` (everything up to the output
 projection; ``out`` a column slice to write into, ``gain`` a scalar folded into the last elementwise step) and the
 matrix ``w_o``, so a block can fuse the projection with the residual add and ``SideBySide`` can run one projection for
 all of its members.
@@ -59,6 +71,13 @@ class StepContext:
     cache: object            # HybridCache (or a row view)
     slot0: object            # int, or device int32[1] (graph-capturable)
     u: Optional[torch.Tensor] = None  # hyper-connected stacks: the next sublayer's input sum, left by the last write
+    # depth-averaging stacks: every layer's result so far [L + 1, M, D]; the next layer's normed input, left by the last
+    # update; the number format of normed inputs and features; whether the step needs the final norm of every row
+    hist: Optional[torch.Tensor] = None
+    h: Optional[torch.Tensor] = None
+    act_dtype: torch.dtype = torch.float32
+    every_row: bool = False
+    v_first: Optional[torch.Tensor] = None  # values [M, G vdim] of the first value-mixing layer of this step
 
 
 class BiasedAttention:
@@ -436,7 +455,8 @@ class RotaryLatentAttention(LatentAttention):
     plain keys and its values are linear maps) followed by ``rot_dim`` numbers rotated by the token's position: one
     rotated key part shared by all heads. Queries come from a latent of their own (down projection, RMS norm with a plain
     gain, up projection) and are laid out per head as ``dim`` plain numbers, then ``rot_dim`` rotated ones; the score is
-    ``(q_plain . k_plain + q_rot . k_rot) * scale``. Rotation pairs number ``2i`` with ``2i + 1``. ``window > 0``: a
+    ``(q_plain . k_plain + q_rot . k_rot) * scale``. Rotation pairs number ``2i`` with ``2i + 1``, or (``interleaved=False``)
+    ``i`` with ``i + rot_dims / 2``. ``window > 0``: a
     query sees the last ``window`` positions (and the first ``keep_first`` of the sequence). Each head's output is
     multiplied by the sigmoid of one more projection of the mixer's input.
 
@@ -447,9 +467,10 @@ class RotaryLatentAttention(LatentAttention):
 
     def __init__(self, layer_idx: int, spec, eps: float, w_in: torch.Tensor, dq_norm: torch.Tensor, w_uq: torch.Tensor,
                  dkv_norm: torch.Tensor, w_uk: torch.Tensor, w_uv: torch.Tensor, freq: Optional[torch.Tensor],
-                 w_o: torch.Tensor, gated: bool = True):
+                 w_o: torch.Tensor, gated: bool = True, interleaved: bool = True):
         self.i = layer_idx
         self.gated = gated        # whether w_in ends with one gate row per head
+        self.interleaved = interleaved
         self.spec = spec
         self.eps = eps
         self.w_in = w_in          # [q_rank + kv_rank + rot_dim (+ H), D]: query latent, key / value latent, rotated key, gates
@@ -468,6 +489,7 @@ class RotaryLatentAttention(LatentAttention):
         wv[:, :, :rank] = w_uv
         self.w_uv_row = wv        # [H, vdim, rank + rot]: a head's values from a cache row
         self.w_uv = w_uv          # [H, vdim, rank]: ... from the attended latent
+        self.head, self.width, self.o_bias = spec.vdim, nh * spec.vdim, None
 
     def expands(self, s: int, n: int, bf16: bool) -> bool:
         sp = self.spec
@@ -483,16 +505,19 @@ class RotaryLatentAttention(LatentAttention):
         return expanded < latent
 
     def __call__(self, h, ctx: StepContext) -> torch.Tensor:
+        return hy.linear(self.features(hy.linear(h, self.w_in), ctx), self.w_o)
+
+    def features(self, proj: torch.Tensor, ctx: StepContext, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         sp = self.spec
         m, nh, rank, rot = ctx.b * ctx.s, sp.heads, sp.kv_rank, sp.rot_dim
         kd, row = sp.dim + rot, rank + rot
-        proj = hy.linear(h, self.w_in)
         c, _ = ctx.cache.layer(self.i)
         cq = hy.latent_rope_prep(proj, 0, self.dq_norm, sp.q_rank, self.dkv_norm, self.freq, ctx.positions, ctx.slot0,
-                                 ctx.b, ctx.s, c, self.eps)
+                                 ctx.b, ctx.s, c, self.eps, self.interleaved,
+                                 torch.bfloat16 if hy.prompt_bf16(m, sp.q_rank, self.w_uq.dtype) else torch.float32)
         q = hy.linear(cq, self.w_uq)
         if self.freq is not None:
-            hy.rotate_heads(q, ctx.positions, self.freq, nh, out=q, offset=sp.dim, interleaved=True)
+            hy.rotate_heads(q, ctx.positions, self.freq, nh, out=q, offset=sp.dim, interleaved=self.interleaved)
         gate = proj[:, sp.q_rank + row:sp.q_rank + row + nh] if self.gated else None
         s0 = ctx.cache.index if torch.is_tensor(ctx.slot0) else int(ctx.slot0)  # (host mirror of the slot)
         n = s0 + ctx.s
@@ -505,14 +530,12 @@ class RotaryLatentAttention(LatentAttention):
             first = max(0, s0 - sp.window + 1) // 64 * 64 if sp.window and not sp.keep_first else 0
             k = hy.latent_expand(c, n, self.w_uk, first)
             v = hy.latent_expand(c, n, self.w_uv_row, first)
-            o = hy.attn_bias(q.reshape(ctx.b, ctx.s, nh, kd), k, v, ctx.slot0 if first == 0 else s0 - first, sp.scale,
-                             window=sp.window, keep_first=sp.keep_first, gate=gate)
-            return hy.linear(o, self.w_o)
+            return hy.attn_bias(q.reshape(ctx.b, ctx.s, nh, kd), k, v, ctx.slot0 if first == 0 else s0 - first, sp.scale,
+                                window=sp.window, keep_first=sp.keep_first, gate=gate, out=out)
         ql = hy.heads_linear(q.reshape(m, nh, kd), self.w_qk)
         a = hy.attn_bias(ql.reshape(ctx.b, ctx.s, nh, row), c, c, ctx.slot0, sp.scale, window=sp.window,
                          keep_first=sp.keep_first, gate=gate, vdim=rank)
-        o = hy.heads_linear(a.reshape(m, nh, rank), self.w_uv)
-        return hy.linear(o.reshape(m, nh * sp.vdim), self.w_o)
+        return hy.heads_linear(a.reshape(m, nh, rank), self.w_uv, out).reshape(m, nh * sp.vdim)
 
 
 class NormedGatedAttention:
@@ -606,3 +629,133 @@ class HyperBlock:
             u = hy.hc_update_(xs, self.hc2[1], self.hc2[2], f.y, f.nsum, f.row_w, f.row_expert, f.n_real, f.ident, f.extra,
                               next_in=self.next_in)
         ctx.u = u
+
+
+class WholeNormAttention:
+    """Softmax attention over this layer's own keys and values: one bias per q / k / v column; q and k RMS-normed over the
+    WHOLE projection (all heads at once) with a gain per column; rotary positions on the first ``2 len(freq)`` numbers of
+    every head (pairs ``2i``, ``2i + 1``); ``window > 0``: a query sees the last ``window`` positions; a per-head sink in the
+    softmax denominator (zeros: a constant one beside the exponentials). ``lam``: the values are blended with the first
+    value-mixing layer's of the same token before they are cached, ``v <- (1 - lam) v + lam v_first``; that first layer
+    (``lam`` None, ``leads``) leaves its values in the step's context. ``gated``: every output column is multiplied by the
+    sigmoid of a projection column of its own. The output projection's bias is ``o_bias``."""
+
+    def __init__(self, layer_idx: int, spec, eps: float, w_in: torch.Tensor, bias: Optional[torch.Tensor],
+                 q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], freq: Optional[torch.Tensor],
+                 sink: Optional[torch.Tensor], leads: bool, lam: Optional[torch.Tensor], w_o: torch.Tensor,
+                 o_bias: Optional[torch.Tensor], gated: bool = True, interleaved: bool = True):
+        self.i = layer_idx
+        self.spec = spec
+        self.eps = eps
+        self.w_in = w_in    # [H dim + G dim + G vdim (+ H vdim), D]: q | k | v | gates
+        self.bias = bias    # fp32 [H dim + G dim + G vdim] or None
+        self.q_norm, self.k_norm = q_norm, k_norm  # fp32 [H dim], [G dim]
+        self.freq = freq    # float64 [rot_dims / 2] or None
+        self.sink = sink    # fp32 [H] or None
+        self.leads, self.lam = leads, lam
+        self.gated, self.interleaved = gated, interleaved
+        self.w_o, self.o_bias = w_o, o_bias  # [D, H vdim], fp32 [D] or None
+        self.head, self.width = spec.vdim, spec.heads * spec.vdim
+
+    def features(self, proj: torch.Tensor, ctx: StepContext, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        sp = self.spec
+        kc, vc = ctx.cache.layer(self.i)
+        q, v = hy.qkv_prep(proj, self.bias, self.q_norm, self.k_norm, self.eps, ctx.positions, ctx.slot0, ctx.b, ctx.s,
+                           sp.heads, sp.kv_heads, sp.dim, sp.vdim, kc, vc, self.freq, self.interleaved,
+                           ctx.v_first if self.lam is not None else None, self.lam, self.leads)
+        if self.leads:
+            ctx.v_first = v
+        c = (sp.heads + sp.kv_heads) * sp.dim + sp.kv_heads * sp.vdim
+        gate = proj[:, c:c + self.width] if self.gated else None
+        return hy.attn_bias(q, kc, vc, ctx.slot0, sp.scale, sink=self.sink, window=sp.window, gate=gate, gate_cols=True,
+                            out=out)
+
+
+class GatedRunningMixer:
+    """Linear attention over a carried fp32 state whose forget gate also decides what is written. Per head and key channel
+    the gate is ``f = l + (1 - l) sigmoid(W_f h + b_f)`` with a fixed lower bound ``l``; ``S <- diag(f) S + (1 - f) v^T``,
+    ``o = S^T silu(W_q h)``; then each head's ``o`` over its root mean square, times a gain shared by the heads."""
+
+    def __init__(self, layer_idx: int, spec, eps: float, w_in: torch.Tensor, f_bias: torch.Tensor, lower: torch.Tensor,
+                 norm_w: torch.Tensor, w_o: torch.Tensor):
+        self.i = layer_idx
+        self.spec = spec
+        self.eps = eps
+        self.w_in = w_in        # [2 H dim + H vdim, D]: q | f | v
+        self.f_bias = f_bias    # fp32 [H dim]
+        self.room = 1.0 - lower  # fp32 [H dim]: what the gate can give up
+        self.norm_w = norm_w    # fp32 [vdim]
+        self.w_o, self.o_bias = w_o, None  # [D, H vdim]
+        self.head, self.width = spec.vdim, spec.heads * spec.vdim
+
+    def features(self, proj: torch.Tensor, ctx: StepContext, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        sp = self.spec
+        qk, hd = sp.heads * sp.dim, (sp.heads, sp.dim)
+        state, _ = ctx.cache.recurrent(self.i)
+        o = hy.gated_running_scan(proj[:, :qk].unflatten(1, hd), proj[:, 2 * qk:2 * qk + self.width].unflatten(
+            1, (sp.heads, sp.vdim)), proj[:, qk:2 * qk].unflatten(1, hd), self.f_bias, self.room, state, ctx.b, ctx.s)
+        return hy.gated_rmsnorm(o, None, self.norm_w, self.eps, hy.GATE_NONE, out=out)
+
+
+class GatedMoE:
+    """The routed part of a mixture of gated experts: ``top`` of ``experts`` chosen by a grouped router (``rule``), each
+    weighted on its OUTPUT. The router's rows are part of the block's fused input product; a shared expert is the block's
+    dense side."""
+
+    def __init__(self, experts: int, top: int, groups: int, keep: int, rule, w_router: torch.Tensor, w_gu: torch.Tensor,
+                 w_down: torch.Tensor, act: int = hy.ACT_SWIGLU):
+        self.experts, self.top, self.groups, self.keep, self.rule, self.act = experts, top, groups, keep, rule, act
+        self.w_router = w_router  # [E, D]
+        self.w_gu = w_gu          # [E, 2 ff, D] gate rows then up rows
+        self.w_down = w_down      # [E, D, ff]
+
+    def __call__(self, h: torch.Tensor, z: torch.Tensor):
+        """``(y [M * top, D] unweighted, row_w [M * top])`` for the router logits ``z [M, E]``."""
+        y, _, row_w = hy.moe_grouped(h, z, None, self.top, self.groups, self.keep, self.w_gu, self.w_down, self.act, self.rule)
+        return y, row_w
+
+
+class DepthAverageBlock:
+    """``h = norm(x); X_(i+1) = x + mult * (mixer(h) + ff(h)); x <- sum_{j <= i+1} coef[j] X_j``: mixer and feed-forward read
+    one normed input, and what goes on is a weighted sum of every layer's result so far (``X_0``: the embedding).
+
+    One product serves the mixer's input projection and the router; the mixer's features and the dense side's activation (a
+    dense feed-forward or a shared expert, ``side_gu`` / ``side_down``) lie side by side in front of one output product; the
+    residual add, the mixture's weighted sum, the depth average and the next layer's norm are one elementwise kernel."""
+
+    def __init__(self, i: int, mixer, moe: Optional[GatedMoE], side_gu: Optional[torch.Tensor],
+                 side_down: Optional[torch.Tensor], side_act: int, norm, coef: torch.Tensor, mult: float):
+        self.i, self.mixer, self.moe, self.side_act, self.norm, self.mult = i, mixer, moe, side_act, norm, mult
+        self.coef = coef        # fp32 [i + 2]
+        self.side_gu = side_gu  # [2 ff, D] or None
+        self.side_ff = side_gu.shape[0] // 2 if side_gu is not None else 0
+        self.w_out = mixer.w_o if side_down is None else torch.cat([mixer.w_o, side_down], 1).contiguous()
+        rows = [mixer.w_in] + ([moe.w_router.to(mixer.w_in.dtype)] if moe is not None else [])
+        self.z0 = mixer.w_in.shape[0]
+        n = sum(r.shape[0] for r in rows)
+        if n % 16:  # (whole 16-row tiles, which the packed GEMM takes)
+            rows.append(torch.zeros(16 - n % 16, mixer.w_in.shape[1], dtype=mixer.w_in.dtype, device=mixer.w_in.device))
+        self.w_in = torch.cat(rows, 0).contiguous() if len(rows) > 1 else mixer.w_in
+        mixer.w_in = mixer.w_o = None  # (held once, in the fused matrices)
+        if moe is not None:
+            moe.w_router = None
+        self.next_norm = None   # what the next layer (or the model's end) reads x through
+        self.last = False
+
+    def __call__(self, x: torch.Tensor, ctx: StepContext) -> None:
+        h = ctx.h
+        proj = hy.linear(h, self.w_in)
+        widths = [self.mixer.width] + ([self.side_ff] if self.side_ff else [])
+        feats, *parts = hy.feature_rows(h.shape[0], widths, self.mixer.head, h.dtype, h.device)
+        self.mixer.features(proj, ctx, parts[0])
+        if self.side_ff:
+            hy.linear_glu(h, self.side_gu, self.side_act, parts[1])
+        y = hy.linear(feats, self.w_out)
+        ye = row_w = None
+        if self.moe is not None:
+            ye, row_w = self.moe(h, proj[:, self.z0:self.z0 + self.moe.experts])
+        # (a prompt whose last token alone is wanted norms that row at the end)
+        norm = self.next_norm if not self.last or ctx.every_row else None
+        ctx.h = hy.depth_update_(ctx.hist, self.i, ctx.hist[0] if self.i == 0 else x, x, self.mult, y, self.coef,
+                                 self.mixer.o_bias, ye, self.moe.top if self.moe is not None else 1, row_w, not self.last,
+                                 norm, ctx.act_dtype)

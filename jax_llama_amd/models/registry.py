@@ -43,12 +43,18 @@ def _zifisun():
     return ZifisunConfig, ZifisunForCausalLM
 
 
+def _fokisun():
+    from ..config import FokisunConfig
+    from .fokisun import FokisunForCausalLM
+    return FokisunConfig, FokisunForCausalLM
+
+
 # architecture name (lower case) -> () -> (config class, model class)
 MODEL_REGISTRY: Dict[str, Callable[[], Tuple[type, type]]] = {"llama": _llama, "zavevik": _zavevik,
                                                               "zasevik": _zasevik, "besulix": _besulix,
-                                                              "zifisun": _zifisun}
+                                                              "zifisun": _zifisun, "fokisun": _fokisun}
 # families on the layer-list step function (models/layer_list.py): both number formats, the hybrid extension
-LAYER_LIST_FAMILIES = ("zavevik", "zasevik", "besulix", "zifisun")
+LAYER_LIST_FAMILIES = ("zavevik", "zasevik", "besulix", "zifisun", "fokisun")
 
 
 def register(name: str, factory: Callable[[], Tuple[type, type]]) -> None:

@@ -29,8 +29,15 @@ Mechanisms (each with its constants as arguments, usable by any model of the reg
     sigmoid gate per (token, head) on the output, values that are the leading columns of the key rows;
     ``attn_prep(q_w=, k_w=, norm_v=)``: weighted per-head q / k norms; ``latent_rope_prep`` + ``rotate_heads(offset=,
     interleaved=)``: latent attention with a normed query latent and one rotated key part shared by all heads;
-  * ``route_grouped`` / ``moe_grouped``: softmax-score router with a selection bias, expert groups and identity
-    experts; ``hc_in`` / ``hc_update_``: several residual streams mixed around every sublayer (hyper-connections).
+  * ``route_grouped`` / ``moe_grouped``: softmax- or sigmoid-score router with a selection bias, expert groups (scored
+    by their largest or their two largest members), optionally renormalised and scaled weights, and identity experts;
+    ``hc_in`` / ``hc_update_``: several residual streams mixed around every sublayer (hyper-connections);
+  * ``qkv_prep`` + ``attn_bias(gate_cols=, out=)``: q / k norms over the whole projection, rotary positions in either pair
+    layout, values blended with another layer's, a gate per output column; ``gated_running_scan``: linear attention whose
+    forget gate also decides what is written (``lin_scan`` mode 2);
+  * ``squash_rows`` / ``depth_update_``: a statistics-free norm (``tanh(alpha x) w + b``) and the residual step of a stack
+    whose layers read a weighted sum of every earlier layer's result; ``linear_glu``: gated feed-forward halves written
+    into a column slice, so that several sublayers' features share one output product.
 """
 from __future__ import annotations
 
@@ -48,7 +55,7 @@ F32 = torch.float32
 ATTN_MAX_HEAD = 512
 ATTN_MAX_KEY = 1024
 # epilogues of a row linear (csrc/hybrid/hybrid.h RowAct)
-ACT_NONE, ACT_RELU2, ACT_SWIGLU, ACT_CLAMP_GLU, ACT_SOFTCAP = 0, 1, 2, 3, 4
+ACT_NONE, ACT_RELU2, ACT_SWIGLU, ACT_CLAMP_GLU, ACT_SOFTCAP, ACT_GELU_GLU = 0, 1, 2, 3, 4, 5
 
 _EXT = None
 _ERR: Optional[BaseException] = None
@@ -104,15 +111,19 @@ def _round_like(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 # ------------------------------------------------------------------------------------------------ rows
 def embed_rows(ids: torch.Tensor, table: torch.Tensor, col0: int = 0, ncols: Optional[int] = None,
-               scale: float = 1.0, copies: int = 1) -> torch.Tensor:
+               scale: float = 1.0, copies: int = 1, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """fp32 ``[M, ncols]`` = ``table[ids, col0 : col0 + ncols] * scale``; ``copies > 1``: ``[copies, M, ncols]``, the
-    same rows ``copies`` times (the residual streams of a hyper-connected stack all start from the embedding)."""
+    same rows ``copies`` times (the residual streams of a hyper-connected stack all start from the embedding). ``out``
+    (one copy): a contiguous ``[M, ncols]`` tensor to write into."""
     ncols = table.shape[1] - col0 if ncols is None else ncols
     ids = ids.reshape(-1)
     if not _gpu(table):
         x = table[ids.long(), col0:col0 + ncols].float() * torch.tensor(scale, dtype=F32)
+        if out is not None:
+            return out.copy_(x)
         return x if copies == 1 else x[None].repeat(copies, 1, 1)
-    out = torch.empty(copies * ids.numel(), ncols, dtype=F32, device=table.device)
+    if out is None:
+        out = torch.empty(copies * ids.numel(), ncols, dtype=F32, device=table.device)
     ext().embed_rows(ids.to(torch.int32).contiguous(), table, int(col0), out, float(scale), int(copies))
     return out if copies == 1 else out.reshape(copies, ids.numel(), ncols)
 
@@ -181,7 +192,7 @@ def _fuse_norm(x, rows: int, n: int):
 
 
 def act_gated(act: int) -> bool:
-    return act in (ACT_SWIGLU, ACT_CLAMP_GLU)
+    return act in (ACT_SWIGLU, ACT_CLAMP_GLU, ACT_GELU_GLU)
 
 
 def _act_cpu(y: torch.Tensor, act: int, limit: float, alpha: float) -> torch.Tensor:
@@ -196,6 +207,8 @@ def _act_cpu(y: torch.Tensor, act: int, limit: float, alpha: float) -> torch.Ten
     g, u = y[..., :n], y[..., n:]
     if act == ACT_SWIGLU:
         return torch.nn.functional.silu(g) * u
+    if act == ACT_GELU_GLU:
+        return gelu_tanh(g) * u
     g = g.clamp(max=limit)
     return g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + 1.0)
 
@@ -205,8 +218,9 @@ def linear(x, w: torch.Tensor, swiglu: bool = False, act: int = ACT_NONE, limit:
     """``act(x [M, K] (fp32, or an ``RmsInput``) @ w^T)`` -> fp32 ``[M, N]``. ``act``: none, ``ACT_RELU2`` (``max(y, 0)^2``),
     ``ACT_SOFTCAP`` (``limit * tanh(y / limit)``; ``limit = 1`` is a plain tanh), or a gated
     form for which ``w`` is ``[2N, K]`` (gate rows, then up rows): ``ACT_SWIGLU`` (``silu(g) * u``; also
-    ``swiglu=True``) or ``ACT_CLAMP_GLU`` (``g' sigmoid(alpha g') (u' + 1)``, ``g' = min(g, limit)``,
-    ``u' = clamp(u, -limit, limit)``). ``x`` may be a column-contiguous view with strided rows."""
+    ``swiglu=True``), ``ACT_GELU_GLU`` (``gelu_tanh(g) * u``) or ``ACT_CLAMP_GLU`` (``g' sigmoid(alpha g') (u' + 1)``,
+    ``g' = min(g, limit)``, ``u' = clamp(u, -limit, limit)``). ``x`` may be a column-contiguous view with strided rows; with
+    bf16 weights and no activation it may be bf16 already (the operand it would be rounded to anyway)."""
     if swiglu:
         act = ACT_SWIGLU
     n = w.shape[0] // 2 if act_gated(act) else w.shape[0]
@@ -215,13 +229,55 @@ def linear(x, w: torch.Tensor, swiglu: bool = False, act: int = ACT_NONE, limit:
         return _act_cpu(_round_like(x, w) @ w.float().t(), act, limit, alpha)
     if act == ACT_NONE and norm_w is None and _use_packed_gemm(x, w):
         from . import linear as packed_linear
-        xb = torch.empty(x.shape, dtype=BF16, device=x.device)
-        ext().cast_bf16(x, xb)
-        return packed_linear(xb, _packed_weight(w), out_dtype=F32)
+        return packed_linear(_bf16_rows(x), _packed_weight(w), out_dtype=F32)
     out = torch.empty(x.shape[0], n, dtype=F32, device=x.device)
     ext().linear_rows(x, None, w, out, None, None, None, x.shape[0], int(act), float(limit), float(alpha), None, norm_w,
                       norm_eps)
     return out
+
+
+def _bf16_rows(x: torch.Tensor) -> torch.Tensor:
+    """``x`` as the bf16 operand of a packed GEMM."""
+    if x.dtype == BF16:
+        return x
+    xb = torch.empty(x.shape, dtype=BF16, device=x.device)
+    ext().cast_bf16(x, xb)
+    return xb
+
+
+def prompt_bf16(m: int, cols: int, wdtype) -> bool:
+    """Whether a step of ``m`` rows keeps a sublayer's input and features in bf16 (the matrix operands they would be
+    rounded to anyway, half the traffic): prompt-sized batches with bf16 weights. Fewer rows run GEMVs, which read fp32."""
+    return wdtype == BF16 and m >= PACKED_GEMM_MIN_M and cols % 8 == 0
+
+
+def linear_glu(x: torch.Tensor, w: torch.Tensor, act: int, out: torch.Tensor, limit: float = 0.0,
+               alpha: float = 1.0) -> torch.Tensor:
+    """``out [M, F] = act(x @ w[:F]^T, x @ w[F:]^T)`` for a gated activation; ``out`` may be a column slice of a wider
+    buffer and has ``x``'s type (fp32, or bf16 for the operands of a prompt's next product). A prompt-sized bf16 batch runs
+    the product on the packed MFMA GEMM and the activation as one elementwise pass that writes the slice; otherwise the
+    row linear with the activation in its epilogue."""
+    if not _gpu(x):
+        return out.copy_(_act_cpu(_round_like(x, w) @ w.float().t(), act, limit, alpha))
+    if _use_packed_gemm(x, w):
+        from . import linear as packed_linear
+        ext().glu_rows(packed_linear(_bf16_rows(x), _packed_weight(w), out_dtype=F32), out, int(act), float(limit),
+                       float(alpha))
+        return out
+    ext().linear_rows(x, None, w, out, None, None, None, x.shape[0], int(act), float(limit), float(alpha), None, None, 0.0)
+    return out
+
+
+def feature_rows(m: int, widths, head: int, dtype, device) -> list:
+    """One ``[m, sum(widths)]`` buffer (its rows padded to a multiple of ``head`` numbers, the head size of the first
+    member, so that per-head products can write their rows into it) and its column slices."""
+    n = sum(widths)
+    full = torch.empty(m, -(-n // head) * head, dtype=dtype, device=device)
+    parts, c = [full[:, :n]], 0
+    for wd in widths:
+        parts.append(full[:, c:c + wd])
+        c += wd
+    return parts
 
 
 def ff_dense(x, w_up: torch.Tensor, w_down: torch.Tensor, act: int = ACT_RELU2) -> torch.Tensor:
@@ -262,31 +318,48 @@ def linear_add_(res: torch.Tensor, x, w: torch.Tensor) -> torch.Tensor:
 _HEAD_INDEX = {}
 
 
-def _head_index(m: int, h: int, device) -> Tuple[torch.Tensor, torch.Tensor]:
+def _head_index(m: int, h: int, device, pitch: Optional[int] = None) -> Tuple[torch.Tensor, torch.Tensor]:
     """Index sets that run a per-head linear as an expert-grouped one: linear row ``p = head * m + token`` reads and
-    writes row ``token * h + head``; ``offs[head] = head * m``. Made once per (tokens, heads) and kept (a captured
-    decode step replays with the same tensors)."""
-    key = (m, h, str(device))
+    writes row ``token * pitch + head`` (``pitch``: head rows from one token to the next, ``h`` by default);
+    ``offs[head] = head * m``. Made once per (tokens, heads, pitch) and kept (a captured decode step replays with the
+    same tensors)."""
+    pitch = h if pitch is None else pitch
+    key = (m, h, pitch, str(device))
     got = _HEAD_INDEX.get(key)
     if got is None:
         if len(_HEAD_INDEX) > 4096:
             _HEAD_INDEX.clear()
-        rows = (torch.arange(m, dtype=torch.int32)[None, :] * h + torch.arange(h, dtype=torch.int32)[:, None]).reshape(-1)
+        rows = (torch.arange(m, dtype=torch.int32)[None, :] * pitch + torch.arange(h, dtype=torch.int32)[:, None]).reshape(-1)
         offs = torch.arange(h + 1, dtype=torch.int32) * m
         got = _HEAD_INDEX[key] = (rows.to(device), offs.to(device))
     return got
 
 
-def heads_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+def heads_linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per-head linear: ``x [M, H, K]`` (fp32), ``w [H, N, K]`` -> fp32 ``[M, H, N]``, head ``h`` of every token times
-    ``w[h]^T``. Runs the expert-grouped row linear with the heads as its experts."""
+    ``w[h]^T``. Runs the expert-grouped row linear with the heads as its experts. ``out``: the first ``H * N`` columns of a
+    buffer whose rows are a multiple of ``N`` wide (``feature_rows``), fp32 or (more than ``GROUPED_GEMV_MAX_R`` rows) bf16;
+    returned as it is."""
     m, h, k = x.shape
     n = w.shape[1]
     if not _gpu(x):
-        return torch.einsum("mhk,hnk->mhn", _round_like(x, w), w.float())
+        y = torch.einsum("mhk,hnk->mhn", _round_like(x, w), w.float())
+        return y if out is None else out.copy_(y.reshape(m, h * n))
     x2 = x.reshape(m * h, k)
-    out = torch.empty(m * h, n, dtype=F32, device=x.device)
     e = ext()
+    if out is not None:
+        pitch = out.stride(0) if m > 1 else h * n
+        if pitch % n:  # (rows that are no whole number of heads apart: through a dense copy)
+            return out.copy_(heads_linear(x, w).reshape(m, h * n))
+        dst = torch.as_strided(out, ((m - 1) * (pitch // n) + h, n), (n, 1))
+        src_rows, offs = _head_index(m, h, x.device)
+        if m == 1 and h <= e.GEMV_MAX_R and out.dtype == F32:
+            e.linear_rows(x2, None, w, dst, None, None, src_rows, h, ACT_NONE, 0.0, 1.0, None, None, 0.0)
+        else:
+            e.linear_rows(x2, src_rows, w, dst, _head_index(m, h, x.device, pitch // n)[0], offs, None, m * h, ACT_NONE,
+                          0.0, 1.0, None, None, 0.0, m)
+        return out
+    out = torch.empty(m * h, n, dtype=F32, device=x.device)
     if m == 1 and h <= e.GEMV_MAX_R:  # one token: a GEMV per head
         rows, _ = _head_index(1, h, x.device)
         e.linear_rows(x2, None, w, out, None, None, rows, h, ACT_NONE, 0.0, 1.0, None, None, 0.0)
@@ -428,40 +501,58 @@ def moe_routed(x, z: torch.Tensor, top: int, w_gu: torch.Tensor, w_down: torch.T
     return y
 
 
-def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1):
-    """Softmax-score router over logits ``z [M, E]`` (fp32): scores ``s = softmax(z)``; the choice is made on
+class RouterRule:
+    """How a grouped router turns logits into choices and weights: ``sigmoid`` scores (else softmax), ``group_top`` the
+    number of largest scores summed into a group's score (1 or 2), ``normalise`` the chosen scores to sum 1, ``scale``
+    the weights by a constant. The default is ``route_grouped``'s plain softmax rule."""
+
+    def __init__(self, sigmoid: bool = False, group_top: int = 1, normalise: bool = False, scale: float = 1.0):
+        if group_top not in (1, 2):
+            raise ValueError("a group's score sums its one or two largest scores")
+        self.sigmoid, self.group_top, self.normalise, self.scale = bool(sigmoid), group_top, bool(normalise), float(scale)
+
+
+SOFTMAX_RULE = RouterRule()
+
+
+def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
+                  rule: RouterRule = SOFTMAX_RULE):
+    """Router over logits ``z [M, E]`` (fp32): scores ``s = softmax(z)`` (or ``sigmoid(z)``); the choice is made on
     ``s + correction`` (``correction [E]``, a selection bias that does not enter the weights); the experts form
-    ``groups`` equal groups of neighbours, a group's score is its largest choice score, and only experts of the ``keep``
-    best groups can be chosen (ties to the lower index everywhere); the ``top`` largest are chosen, weight ``s`` of each
-    (not renormalised). Returns ``(row_expert [R], row_w [R])`` in (token, choice) order."""
+    ``groups`` equal groups of neighbours, a group's score is its largest choice score (or its two largest summed), and
+    only experts of the ``keep`` best groups can be chosen (ties to the lower index everywhere); the ``top`` largest are
+    chosen, weight ``s`` of each, renormalised and scaled as ``rule`` says. Returns ``(row_expert [R], row_w [R])`` in
+    (token, choice) order."""
     zz = z.float()
     m, e_n = zz.shape
-    sc = torch.softmax(zz, -1)
+    sc = torch.sigmoid(zz) if rule.sigmoid else torch.softmax(zz, -1)
     ch = sc + correction.float().reshape(1, -1) if correction is not None else sc.clone()
     if groups > 1:
         per = e_n // groups
-        gs = ch.reshape(m, groups, per).max(-1).values
+        gs = ch.reshape(m, groups, per).sort(-1, descending=True).values[..., :rule.group_top].sum(-1)
         best = torch.sort(gs, dim=-1, descending=True, stable=True).indices[:, :keep]
         allowed = torch.zeros(m, groups, dtype=torch.bool).scatter_(1, best, True)
         ch = ch.masked_fill(~allowed.repeat_interleave(per, 1), float("-inf"))
     order = torch.sort(ch, dim=-1, descending=True, stable=True).indices[:, :top]
-    return order.reshape(-1), torch.gather(sc, 1, order).reshape(-1)
+    wt = torch.gather(sc, 1, order)
+    if rule.normalise:
+        wt = wt / (wt.sum(-1, keepdim=True) + 1e-20)
+    return order.reshape(-1), (wt * rule.scale).reshape(-1)
 
 
 def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int,
-                w_up: torch.Tensor, w_down: torch.Tensor, act: int = ACT_RELU2):
+                w_up: torch.Tensor, w_down: torch.Tensor, act: int = ACT_RELU2, rule: RouterRule = SOFTMAX_RULE):
     """Experts of a ``route_grouped`` mixture: ``z [M, E + I]`` holds the logits of the ``E = w_up.shape[0]`` real
     experts and of ``I`` identity experts behind them (an identity expert returns its input; it has no weights and runs
-    no product). ``w_up [E, F, K]``, ``w_down [E, D, F]``, one-accumulator activation ``act``. Returns
+    no product). ``w_up [E, F, K]``, or for a gated activation ``act`` ``[E, 2F, K]`` (gate rows, then up rows),
+    ``w_down [E, D, F]``; ``z`` may be columns of a fused projection, ``x`` bf16 (a prompt's operand). Returns
     ``(y [M * top, D], row_expert [M * top], row_w [M * top])`` in (token, choice) order: ``y`` rows of real experts hold
     ``W_down act(W_up x)`` unweighted, rows whose expert is ``>= E`` hold nothing (the caller's ``hc_update_`` puts the
     weighted sum together)."""
     m, e_n, e_all = x.shape[0], w_up.shape[0], z.shape[1]
     r = m * top
-    if act_gated(act):
-        raise ValueError("moe_grouped: one-accumulator activations only")
     if not _gpu(x):
-        ex, wt = route_grouped(z, correction, top, groups, keep)
+        ex, wt = route_grouped(z, correction, top, groups, keep, rule)
         xr = _round_like(x.float(), w_up).repeat_interleave(top, 0)
         y = torch.zeros(r, w_down.shape[1], dtype=F32)
         for e in ex.unique().tolist():
@@ -478,22 +569,24 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
     wts = torch.empty(2 * r, dtype=F32, device=dev)
     row_w, sort_w = wts[:r], wts[r:]
     y = torch.empty(r, w_down.shape[1], dtype=F32, device=dev)
-    f = w_up.shape[1]
+    f = w_up.shape[1] // 2 if act_gated(act) else w_up.shape[1]
+    how = (rule.sigmoid, rule.group_top, rule.normalise, rule.scale)
     if r <= e.GEMV_MAX_R:  # decode: one GEMV per (token, choice) row; rows of identity experts are skipped on the device
-        e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, None, None, None, None)
+        e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, None, None, None, None, *how)
         h = torch.empty(r, f, dtype=F32, device=dev)
         e.linear_rows(x, row_tok, w_up, h, None, None, row_expert, r, int(act), 0.0, 1.0, None, None, 0.0)
         e.linear_rows(h, None, w_down, y, None, None, row_expert, r, ACT_NONE, 0.0, 1.0, None, None, 0.0)
     else:
         # expert-grouped over the sorted rows; identity experts sort behind the real ones, past the last offset the
         # linears look at
-        e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, sort_tok, sort_dst, sort_w, offs)
+        e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, sort_tok, sort_dst, sort_w, offs,
+                        *how)
         # with bf16 weights the tiles read a bf16 copy of x and keep the hidden activation bf16 (the operands they would
         # round to anyway): half the activation traffic of both products
         keep_bf16 = w_up.dtype == BF16 and r > GROUPED_GEMV_MAX_R
         h = torch.empty(r, f, dtype=BF16 if keep_bf16 else F32, device=dev)
         xa = x
-        if keep_bf16 and x.is_contiguous() and x.numel() % 8 == 0:
+        if keep_bf16 and x.dtype == F32 and x.is_contiguous() and x.numel() % 8 == 0:
             xa = torch.empty(x.shape, dtype=BF16, device=dev)
             e.cast_bf16(x, xa)
         e.linear_rows(xa, sort_tok, w_up, h, None, offs, None, r, int(act), 0.0, 1.0, None, None, 0.0)
@@ -542,6 +635,49 @@ def hc_update_(xs: torch.Tensor, mix: torch.Tensor, out_w: torch.Tensor, y: torc
     u = torch.empty(m, d, dtype=F32, device=xs.device) if next_in is not None else None
     ext().hc_update(xs, mix, out_w, y, int(nsum), row_w, row_expert, int(n_real), ident, extra, next_in, u)
     return u
+
+
+class SquashNorm:
+    """A norm without statistics: ``tanh(alpha * x) * w + b`` (``alpha`` one number, ``w`` and ``b`` ``[D]``, all fp32)."""
+
+    def __init__(self, alpha: torch.Tensor, w: torch.Tensor, b: torch.Tensor):
+        self.alpha, self.w, self.b = alpha.reshape(1), w.reshape(-1), b.reshape(-1)
+
+
+def squash_rows(x: torch.Tensor, norm: SquashNorm, dtype=F32) -> torch.Tensor:
+    """``tanh(alpha * x) * w + b`` for ``x [M, D]`` (fp32) -> fp32 or bf16 ``[M, D]``."""
+    if not _gpu(x):
+        return (torch.tanh(norm.alpha * x.float()) * norm.w + norm.b).to(dtype)
+    h = torch.empty(x.shape, dtype=dtype, device=x.device)
+    ext().squash_rows(x, norm.alpha, norm.w, norm.b, h)
+    return h
+
+
+def depth_update_(hist: torch.Tensor, i: int, x: torch.Tensor, x_out: torch.Tensor, mult: float, y: torch.Tensor,
+                  coef: torch.Tensor, bias: Optional[torch.Tensor] = None, ye: Optional[torch.Tensor] = None, nsum: int = 1,
+                  row_w: Optional[torch.Tensor] = None, store: bool = True, norm: Optional[SquashNorm] = None,
+                  h_dtype=F32) -> Optional[torch.Tensor]:
+    """One residual step of a stack that averages over its depth. ``hist [planes, M, D]`` (fp32) holds ``X_0 .. X_i``:
+    ``X = x + mult * (y + bias + sum_c row_w[m * nsum + c] ye[m * nsum + c])`` is written to ``hist[i + 1]`` (``store``), and
+    ``x_out`` (may be ``x``) becomes ``coef[i + 1] X + sum_{j <= i} coef[j] hist[j]``. ``norm``: also returns the next
+    layer's input ``tanh(alpha x_out) w + b`` (fp32 or bf16)."""
+    if not _gpu(x):
+        v = y.float()
+        if bias is not None:
+            v = v + bias
+        if ye is not None:
+            m = v.shape[0]
+            v = v + (ye.float().reshape(m, nsum, -1) * row_w.float().reshape(m, nsum, 1)).sum(1)
+        new = x.float() + mult * v
+        if store:
+            hist[i + 1].copy_(new)
+        x_out.copy_((hist[:i + 1] * coef[:i + 1, None, None]).sum(0) + coef[i + 1] * new)
+        return squash_rows(x_out, norm, h_dtype) if norm is not None else None
+    h = torch.empty(x.shape, dtype=h_dtype, device=x.device) if norm is not None else None
+    ext().depth_update(hist, int(i), bool(store), x, x_out, float(mult), y, bias, ye, int(nsum), row_w, coef,
+                       norm.alpha if norm is not None else None, norm.w if norm is not None else None,
+                       norm.b if norm is not None else None, h)
+    return h
 
 
 def norm_residual_(x: torch.Tensor, y: torch.Tensor, w: torch.Tensor, eps: float, nsum: int = 1, ysc: float = 1.0,
@@ -678,14 +814,15 @@ def latent_prep(proj: torch.Tensor, col0: int, w: torch.Tensor, slot, b: int, s:
 
 def latent_rope_prep(proj: torch.Tensor, q_col0: int, q_w: torch.Tensor, c_col0: int, c_w: torch.Tensor,
                      freq: Optional[torch.Tensor], positions: torch.Tensor, slot, b: int, s: int, cache: torch.Tensor,
-                     eps: float) -> torch.Tensor:
+                     eps: float, interleaved: bool = True, q_dtype=F32) -> torch.Tensor:
     """The step after the fused down projection of a latent attention whose queries go through a latent too and whose
     keys carry one rotated part shared by all heads. From ``proj [B*S, .]``:
-      * columns ``[q_col0, q_col0 + len(q_w))``: RMS-normed, times the plain gain ``q_w`` -> returned dense (fp32), the
-        input of the queries' up projection;
+      * columns ``[q_col0, q_col0 + len(q_w))``: RMS-normed, times the plain gain ``q_w`` -> returned dense (fp32 or bf16),
+        the input of the queries' up projection;
       * columns ``[c_col0, c_col0 + rank)``, ``rank = len(c_w)``: RMS-normed, times ``c_w`` -> ``cache[b, 0, slot + s, :rank]``;
       * the next ``cache.shape[3] - rank`` columns (not normed): their first ``2 len(freq)`` numbers rotated by the
-        token's position, number ``2i`` with number ``2i + 1``, angle ``position * freq[i]`` -> ``cache[..., rank:]``."""
+        token's position, number ``2i`` with number ``2i + 1`` (``interleaved=False``: ``i`` with ``i + len(freq)``), angle
+        ``position * freq[i]`` -> ``cache[..., rank:]``."""
     rank, q_rank = c_w.numel(), q_w.numel()
     nrot = cache.shape[3] - rank
     if not _gpu(proj):
@@ -698,12 +835,12 @@ def latent_rope_prep(proj: torch.Tensor, q_col0: int, q_w: torch.Tensor, c_col0:
         if nrot:
             r = proj[:, c_col0 + rank:c_col0 + rank + nrot].float().reshape(b * s, 1, nrot)
             if freq is not None:
-                r = _turn_pairs_cpu(r, positions.reshape(-1), freq)
+                r = (_turn_pairs_cpu if interleaved else _turn_cpu)(r, positions.reshape(-1), freq)
             cache[:, 0, s0:s0 + s, rank:] = r.reshape(b, s, nrot).to(cache.dtype)
-        return cq.contiguous()
-    cq = torch.empty(b * s, q_rank, dtype=F32, device=proj.device)
+        return cq.to(q_dtype).contiguous()
+    cq = torch.empty(b * s, q_rank, dtype=q_dtype, device=proj.device)
     ext().latent_prep(proj, int(c_col0), c_w, _slot_tensor(slot, proj.device), b, s, cache, float(eps), cq, int(q_col0), q_w,
-                      freq, positions.reshape(-1).to(torch.int32).contiguous())
+                      freq, positions.reshape(-1).to(torch.int32).contiguous(), not interleaved)
     return cq
 
 
@@ -752,7 +889,8 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
               bias: Optional[torch.Tensor] = None, max_kv: Optional[int] = None,
               sink: Optional[torch.Tensor] = None, chunk: int = 0,
               head_scale: Optional[torch.Tensor] = None, window: int = 0, keep_first: int = 0,
-              gate: Optional[torch.Tensor] = None, vdim: Optional[int] = None) -> torch.Tensor:
+              gate: Optional[torch.Tensor] = None, vdim: Optional[int] = None, gate_cols: bool = False,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal attention of ``q [B, S, H, dim]`` (queries at cache slots ``slot + s``) over ``[B, G, T, .]`` caches:
     ``score = q.k * scale``; ``softcap * tanh(score / softcap)`` if ``softcap > 0``; ``+ bias[min(i - j, last), h]``;
     softmax over ``j <= i``, with ``exp(sink[h])`` added to the denominator when ``sink [H]`` is given (a slot without
@@ -761,8 +899,10 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
     ``head_scale [H]``: the score of head ``h`` is also multiplied by ``head_scale[h]`` (before cap and bias).
     ``window > 0``: query ``i`` sees key ``j <= i`` only if ``i - j < window`` or ``j < keep_first`` (the first
     ``keep_first`` slots of a row stay visible to every later query). ``gate [B*S, >= H]`` (a column view is fine): head
-    ``h``'s output of token ``m`` is multiplied by ``sigmoid(gate[m, h])``. ``kc`` and ``vc`` may be one tensor (latent
-    attention); ``vdim``: the values are the first ``vdim`` columns of ``vc``'s rows. Returns fp32 ``[B*S, H*vdim]``."""
+    ``h``'s output of token ``m`` is multiplied by ``sigmoid(gate[m, h])``; with ``gate_cols`` (``gate [B*S, >= H*vdim]``) its
+    column ``c`` by ``sigmoid(gate[m, h * vdim + c])``. ``kc`` and ``vc`` may be one tensor (latent
+    attention); ``vdim``: the values are the first ``vdim`` columns of ``vc``'s rows. Returns fp32 ``[B*S, H*vdim]``, or
+    ``out``, a column slice of a wider fp32 or bf16 buffer."""
     b, s, h, dim = q.shape
     g = kc.shape[1]
     vdim = vc.shape[3] if vdim is None else int(vdim)
@@ -797,9 +937,12 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
             pr = torch.softmax(sc, -1)
         o = torch.einsum("bhst,bhtv->bshv", pr, v)
         if gate is not None:
-            o = o * torch.sigmoid(gate[:, :h].float()).reshape(b, s, h, 1)
-        return o.reshape(b * s, h * vdim)
-    out = torch.empty(b * s, h * vdim, dtype=F32, device=q.device)
+            gn = vdim if gate_cols else 1
+            o = o * torch.sigmoid(gate[:, :h * gn].float()).reshape(b, s, h, gn)
+        o = o.reshape(b * s, h * vdim)
+        return o if out is None else out.copy_(o)
+    if out is None:
+        out = torch.empty(b * s, h * vdim, dtype=F32, device=q.device)
     e = ext()
     t_cap = int(max_kv) if max_kv is not None else kc.shape[2]
     ws, splits, vt = None, 1, None
@@ -813,7 +956,7 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
             vt = torch.empty(nb // 2, dtype=BF16, device=q.device)
     e.attn_bias(q.contiguous(), kc, vc, _slot_tensor(slot, q.device), float(scale), float(softcap or 0.0), bias, out,
                 t_cap, ws, splits, vt, sink, int(chunk or 0), head_scale, int(window or 0), int(keep_first or 0), gate,
-                vdim)
+                vdim, bool(gate_cols))
     return out
 
 
@@ -885,14 +1028,15 @@ def delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta: torch.Te
     return o
 
 
-GATE_SILU, GATE_SIGMOID = 0, 1
+GATE_SILU, GATE_SIGMOID, GATE_NONE = 0, 1, 2
 
 
-def gated_rmsnorm(o: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, eps: float, gate_act: int = GATE_SILU,
+def gated_rmsnorm(o: torch.Tensor, gate: Optional[torch.Tensor], w: torch.Tensor, eps: float, gate_act: int = GATE_SILU,
                   denom_floor: Optional[torch.Tensor] = None, gain: float = 1.0,
                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``o [M, H, vdim] / rms(o) * w * act(gate [M, H*vdim]) * gain`` -> fp32 ``[M, H*vdim]``. ``w``: ``[vdim]`` (one
-    gain vector for every head) or ``[H*vdim]``; ``gate_act``: ``GATE_SILU`` or ``GATE_SIGMOID``. ``denom_floor [M, H]``:
+    gain vector for every head) or ``[H*vdim]``; ``gate_act``: ``GATE_SILU``, ``GATE_SIGMOID`` or ``GATE_NONE`` (``gate`` is
+    None). ``denom_floor [M, H]``:
     ``o`` is ``[M, H, vdim + 1]`` whose last column is a normaliser ``z``; the head's first ``vdim`` numbers are divided
     by ``max(|z|, denom_floor) + 1e-6`` before the norm. ``out``: a ``[M, H*vdim]`` column slice of a wider buffer."""
     m, h, ov = o.shape
@@ -905,6 +1049,8 @@ def gated_rmsnorm(o: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, eps: flo
             x = x[..., :vdim] / (torch.maximum(x[..., vdim].abs(), denom_floor.float().reshape(m, h)) + 1e-6)[..., None]
         x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
         x = x.reshape(m, h * vdim) * (w.float().repeat(h) if w.numel() == vdim and h > 1 else w.float().reshape(-1))
+        if gate_act == GATE_NONE:
+            return out.copy_(x * gain)
         g = gate.float()
         out.copy_(x * (torch.sigmoid(g) if gate_act == GATE_SIGMOID else torch.nn.functional.silu(g)) * gain)
         return out
@@ -973,6 +1119,50 @@ def rope_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], positions: torch
     ext().rope_prep(proj, bias, positions.reshape(-1).to(torch.int32).contiguous(), _slot_tensor(slot, proj.device), b, s,
                     heads, kv_heads, dim, vdim, kc, vc, q, qk_freq, v_freq)
     return q
+
+
+def qkv_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], q_w: Optional[torch.Tensor], k_w: Optional[torch.Tensor],
+             eps: float, positions: torch.Tensor, slot, b: int, s: int, heads: int, kv_heads: int, dim: int, vdim: int,
+             kc: torch.Tensor, vc: torch.Tensor, freq: Optional[torch.Tensor], interleaved: bool = False,
+             v_prev: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None, keep_v: bool = False):
+    """From the fused projection ``proj [B*S, H*dim + G*dim + G*vdim (+ more)]`` (+ ``bias``, one number per q / k / v
+    column): q divided by the root mean square of ALL its columns, times ``q_w [H*dim]`` (None: no norm), k likewise with
+    ``k_w [G*dim]``; then every q / k head rotated by the token's position on its first ``2 len(freq)`` numbers (pairs
+    ``2i``, ``2i + 1`` when ``interleaved``, else ``i``, ``i + len(freq)``; None: no rotation). ``v_prev [B*S, G*vdim]``: v
+    becomes ``(1 - lam) v + lam v_prev`` (``lam``: one fp32 number). k / v are written into the caches ``[B, G, T, .]`` at
+    ``slot + s``. Returns ``(q [B, S, H, dim] fp32, v)``: ``v [B*S, G*vdim]`` the values before their rounding when ``keep_v``,
+    else None."""
+    m = b * s
+    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    if not _gpu(proj):
+        s0 = _slot_int(slot)
+        y = proj[:, :nq + nk + nv].float()
+        if bias is not None:
+            y = y + bias.float()
+
+        def part(c0, n, w, h):
+            x = y[:, c0:c0 + n]
+            if w is not None:
+                x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+            x = x.reshape(m, h, dim)
+            if freq is not None:
+                x = (_turn_pairs_cpu if interleaved else _turn_cpu)(x, positions.reshape(-1), freq)
+            return x
+
+        q, k = part(0, nq, q_w, heads), part(nq, nk, k_w, kv_heads)
+        v = y[:, nq + nk:]
+        if v_prev is not None:
+            v = (1.0 - lam.float()) * v + lam.float() * v_prev.float()
+        kc[:, :, s0:s0 + s] = k.reshape(b, s, kv_heads, dim).permute(0, 2, 1, 3).to(kc.dtype)
+        vc[:, :, s0:s0 + s] = v.reshape(b, s, kv_heads, vdim).permute(0, 2, 1, 3).to(vc.dtype)
+        return q.reshape(b, s, heads, dim).contiguous(), v.contiguous() if keep_v else None
+    dev = proj.device
+    q = torch.empty(b, s, heads, dim, dtype=F32, device=dev)
+    v = torch.empty(m, nv, dtype=F32, device=dev) if keep_v else None
+    ext().qkv_prep(proj, bias, q_w, k_w, float(eps), positions.reshape(-1).to(torch.int32).contiguous(),
+                   _slot_tensor(slot, dev), b, s, heads, kv_heads, dim, vdim, kc, vc, q, freq, not interleaved, v_prev,
+                   lam if v_prev is not None else None, v)
+    return q, v
 
 
 def rotate_heads(a: torch.Tensor, positions: torch.Tensor, freq: Optional[torch.Tensor], heads: int, sign: float = 1.0,
@@ -1113,4 +1303,28 @@ def timemix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, wpre: torch.
     o = torch.empty(m, h, vdim, dtype=F32, device=r.device)
     nseg, seg_len, ws = _scan_segments(b, s, h, dim, vdim, r.device)
     ext().lin_scan(1, r, k, v, wpre, None, w0.reshape(h, dim), u.reshape(h, dim), state, o, b, s, 1.0, nseg, seg_len, ws)
+    return o
+
+
+def gated_running_scan(q: torch.Tensor, v: torch.Tensor, fpre: torch.Tensor, f_bias: torch.Tensor, room: torch.Tensor,
+                       state: torch.Tensor, b: int, s: int) -> torch.Tensor:
+    """Linear attention whose forget gate also decides what is written, read after the write. ``q, fpre [M, H, dim]``
+    (pre-activations), ``v [M, H, vdim]`` (column views are fine), ``f_bias, room [H, dim]``; ``state [B, H, dim, vdim]``
+    (fp32, advanced): with the write factor ``i = room * sigmoid(-(fpre + f_bias))`` -- one minus a forget gate whose lower
+    bound is ``1 - room`` -- ``S <- diag(1 - i) S + i v^T;  o = S^T silu(q)``. Returns ``o [M, H, vdim]``."""
+    m, h, dim = q.shape
+    vdim = v.shape[2]
+    if not _gpu(q):
+        qq = torch.nn.functional.silu(q.float()).reshape(b, s, h, dim)
+        vv = v.float().reshape(b, s, h, vdim)
+        wr = room.float().reshape(h, dim) * torch.sigmoid(-(fpre.float().reshape(b, s, h, dim) + f_bias.float().reshape(h, dim)))
+        o = torch.empty(b, s, h, vdim)
+        for t in range(s):
+            state.add_(wr[:, t, :, :, None] * (vv[:, t, :, None, :] - state))
+            o[:, t] = torch.einsum("bhdv,bhd->bhv", state, qq[:, t])
+        return o.reshape(m, h, vdim)
+    o = torch.empty(m, h, vdim, dtype=F32, device=q.device)
+    nseg, seg_len, ws = _scan_segments(b, s, h, dim, vdim, q.device)
+    ext().lin_scan(2, q, fpre, v, fpre, None, f_bias.reshape(h, dim), room.reshape(h, dim), state, o, b, s, 1.0, nseg,
+                   seg_len, ws)
     return o
