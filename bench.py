@@ -87,6 +87,9 @@ def main():
     ap.add_argument("--stream-compare", action="store_true", help="the same comparison for the family of windowed latent "
                     "/ normed attention, grouped routing and several residual streams: Zifisun beside Zasevik (the closest "
                     "family) and LLaMA")
+    ap.add_argument("--depth-compare", action="store_true", help="the same comparison for the family that averages over its "
+                    "depth (rotary, latent and running-memory layers, mixer and feed-forward side by side): Fokisun beside "
+                    "Zifisun (the closest family), Besulix (the closest recurrence) and LLaMA")
     ap.add_argument("--hybrid-sizes", nargs="*", default=["2k", "4k"])
     ap.add_argument("--hybrid-families", nargs="*", default=["zavevik", "llama"])
     ap.add_argument("--hybrid-batches", type=int, nargs="*", default=[1, 8])
@@ -96,6 +99,9 @@ def main():
         return _hybrid_compare(args)
     if args.stream_compare:
         args.hybrid_families = ["zifisun", "zasevik", "llama"]
+        return _hybrid_compare(args)
+    if args.depth_compare:
+        args.hybrid_families = ["fokisun", "zifisun", "besulix", "llama"]
         return _hybrid_compare(args)
     if args.recurrent_compare:
         args.hybrid_families = ["besulix", "zavevik", "llama"]

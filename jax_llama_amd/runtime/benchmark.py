@@ -311,10 +311,35 @@ def zifisun_like(width: int, heads: int, kv_heads: int, head_dim: int, ffn: int,
                                     "streams": streams, "layers": ls})
 
 
+def fokisun_like(width: int, heads: int, kv_heads: int, head_dim: int, ffn: int, layers: int, vocab: int,
+                 kv_rank: int = 448, window: int = 1024, experts: int = 8, top: int = 2):
+    """A Fokisun config whose layers have a LLaMA layer's sizes, in turn: attention (``heads`` / ``kv_heads`` heads of
+    ``head_dim``, all of it rotated, a window of ``window``, value mixing) with a dense feed-forward of ``ffn``; latent
+    attention (keys of ``head_dim / 2`` plain + ``head_dim / 2`` rotated numbers, values of ``head_dim``, a latent of
+    ``kv_rank``, a query latent of ``3 kv_rank / 2``), the gated running memory (``heads`` heads of ``head_dim`` channels and
+    values) and attention again, each of these with ``top`` of ``experts`` experts of ``ffn / 4`` in 4 groups of which 2 are
+    kept, plus a shared expert of ``ffn / 2`` (the active width of the dense FFN at top 2)."""
+    from ..config import FokisunConfig
+    half = head_dim // 2
+    att = dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5, mask={"size": window},
+               rot={"base": 1e4, "dims": head_dim, "scaling": {"factor": 2.0}}, v_mix=True)
+    lat = dict(heads=heads, dim=half, rot_dim=half, vdim=head_dim, kv_rank=kv_rank, q_rank=kv_rank * 3 // 2,
+               scale=head_dim ** -0.5, rot={"base": 1e4, "dims": half})
+    rec = dict(heads=heads, dim=head_dim, vdim=head_dim)
+    groups = 4 if experts % 4 == 0 else 1
+    moe = {"kind": "moe", "expert": {"ff": ffn // 4}, "shared": {"ff": ffn // 2},
+           "router": {"experts": experts, "top": top, "scale": 1.5, "groups": {"count": groups, "keep": max(1, groups // 2)}}}
+    turn = [{"type": "attention", "mixer": att, "mlp": {"kind": "dense", "ff": ffn}},
+            {"type": "latent_attention", "mixer": lat, "mlp": moe}, {"type": "hgrn2", "mixer": rec, "mlp": moe},
+            {"type": "attention", "mixer": att, "mlp": moe}]
+    return FokisunConfig.from_dict({"architecture": "Fokisun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                    "residual_mult": 0.5, "logit_scale": 0.5, "layers": [turn[i % 4] for i in range(layers)]})
+
+
 def hybrid_compare(device, sizes=("2k", "4k"), prompt_len: int = 2048, gen_len: int = 64, batches=(1, 8),
                    families=("zavevik", "llama"), progress=lambda m: None) -> Dict[str, object]:
-    """Prefill and decode throughput of the layer-list families (Zavevik, Zasevik, Besulix, Zifisun) beside LLaMA at equal layer sizes
-    (random weights, bf16, synthetic ids), all through the decode engine: ``prefill_tokens_per_sec`` of one warm ``prompt_len``-token prompt per row
+    """Prefill and decode throughput of the layer-list families (Zavevik, Zasevik, Besulix, Zifisun, Fokisun) beside LLaMA at equal
+    layer sizes (random weights, bf16, synthetic ids), all through the decode engine: ``prefill_tokens_per_sec`` of one warm ``prompt_len``-token prompt per row
     and hipGraph-replayed ``decode_ms_per_token`` over ``gen_len`` steps behind it."""
     from ..config import LLaMAConfig
     from ..models.llama import LLaMAForCausalLM
@@ -336,6 +361,9 @@ def hybrid_compare(device, sizes=("2k", "4k"), prompt_len: int = 2048, gen_len: 
             elif family == "zifisun":
                 from ..models.zifisun import ZifisunForCausalLM
                 model = ZifisunForCausalLM(zifisun_like(**sz), device=device, dtype=torch.bfloat16, seed=1)
+            elif family == "fokisun":
+                from ..models.fokisun import FokisunForCausalLM
+                model = FokisunForCausalLM(fokisun_like(**sz), device=device, dtype=torch.bfloat16, seed=1)
             else:
                 cfg = LLaMAConfig(vocab_size=sz["vocab"], hidden_size=sz["width"], intermediate_size=sz["ffn"],
                                   num_hidden_layers=sz["layers"], num_attention_heads=sz["heads"],
