@@ -86,75 +86,108 @@ int hy_rope_prep(const RopePrep& p, hipStream_t s) {
 
 // grid (M, Y), 4 waves. Every workgroup takes the token's two statistics (one read of q | k; a prompt's workgroup does a
 // whole token, a decode step's token is shared by Y of them) and the token's sines and cosines once into LDS (they are the
-// same for every head); the heads are then dealt to the waves.
+// same for every head); the heads' pairs are then dealt to the threads.
 constexpr int QP_MAX_HALF = 512;
+constexpr int QP_UNR = 4;
 template <typename CT>
 __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
-  __shared__ float red[16];
+  __shared__ float red[8];
   __shared__ float cs[QP_MAX_HALF], sn[QP_MAX_HALF];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x;
   const int m = blockIdx.x, b = m / p.S, t = *p.slot + (m - b * p.S);
   const float* row = p.proj + (size_t)m * p.ld;
   const int nq = p.H * p.dim, nk = p.G * p.dim;
   const int pos = p.half > 0 ? p.positions[m] : 0;
-  for (int i = tid; i < p.half; i += 256) ro_sincos(pos, p.freq[i], 1.f, &sn[i], &cs[i]);
-  float rq = 1.f, rk = 1.f;
-  auto stat = [&](int c0, int n) {
-    float ss = 0.f;
-    for (int d0 = 0; d0 < n; d0 += 1024) {
-      float v[4];
+  // both sums of squares in one walk over q | k, eight loads of a thread in flight, and the angle table behind them
+  float sq = 0.f, sk = 0.f;
+  if (p.q_w || p.k_w) {
+    for (int d0 = 0; d0 < nq + nk; d0 += 2048) {
+      float v[8];
 #pragma unroll
-      for (int u = 0; u < 4; ++u) {
-        const int d = c0 + min(d0 + tid + 256 * u, n - 1);
+      for (int u = 0; u < 8; ++u) {
+        const int d = min(d0 + tid + 256 * u, nq + nk - 1);
         v[u] = row[d] + (p.bias ? p.bias[d] : 0.f);
       }
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
-        if (d0 + tid + 256 * u < n) ss = fmaf(v[u], v[u], ss);
+      for (int u = 0; u < 8; ++u) {
+        const int d = d0 + tid + 256 * u;
+        if (d < nq) sq = fmaf(v[u], v[u], sq);
+        else if (d < nq + nk) sk = fmaf(v[u], v[u], sk);
+      }
     }
-    ss = block_sum(ss, red);
-    return 1.f / sqrtf(ss / (float)n + p.eps);
-  };
-  if (p.q_w) rq = stat(0, nq);
-  if (p.k_w) rk = stat(nq, nk);
-  __syncthreads();  // (the angle table is complete)
+  }
+  for (int i = tid; i < p.half; i += 256) ro_sincos(pos, p.freq[i], 1.f, &sn[i], &cs[i]);
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((tid & 63) == 0) {
+    red[tid >> 6] = sq;
+    red[4 + (tid >> 6)] = sk;
+  }
+  __syncthreads();  // (the angle table is complete too)
+  sq = red[0] + red[1] + red[2] + red[3];
+  sk = red[4] + red[5] + red[6] + red[7];
+  const float rq = p.q_w ? 1.f / sqrtf(sq / (float)nq + p.eps) : 1.f;
+  const float rk = p.k_w ? 1.f / sqrtf(sk / (float)nk + p.eps) : 1.f;
   const bool store = t >= 0 && t < p.T;  // (cache full: the write is dropped)
   const float lam = p.v_prev ? *p.lambda : 0.f;
-  for (int item = blockIdx.y * 4 + wave; item < p.H + 2 * p.G; item += gridDim.y * 4) {
-    if (item >= p.H + p.G) {
-      const int g = item - p.H - p.G, c0 = nq + nk + g * p.vdim;
-      const size_t fl = ((size_t)m * p.G + g) * p.vdim;
-      CT* cd = reinterpret_cast<CT*>(p.vc) + (((size_t)b * p.G + g) * p.T + (store ? t : 0)) * p.vdim;
-      for (int d = lane; d < p.vdim; d += 64) {
-        float v = row[c0 + d] + (p.bias ? p.bias[c0 + d] : 0.f);
-        if (p.v_prev) v = (1.f - lam) * v + lam * p.v_prev[fl + d];
-        if (p.v_out) p.v_out[fl + d] = v;
-        if (store) ro_st(cd + d, v);
-      }
-      continue;
+  // q / k: an item is a rotated pair or a number that passes, (dim - half) of them per head; values: one number each. A
+  // thread's items are taken QP_UNR at a time, all of their loads before the first use.
+  const int per = p.dim - p.half, n_qk = (p.H + p.G) * per, n_v = p.G * p.vdim;
+  const int step = gridDim.y * 256, first = blockIdx.y * 256 + tid;
+  for (int i0 = first; i0 < n_qk; i0 += QP_UNR * step) {
+    float u[QP_UNR], v[QP_UNR];
+    int head[QP_UNR], pair[QP_UNR], du[QP_UNR], dv[QP_UNR];
+#pragma unroll
+    for (int k = 0; k < QP_UNR; ++k) {
+      const int idx = min(i0 + k * step, n_qk - 1);
+      head[k] = idx / per;
+      const int i = idx - head[k] * per;
+      pair[k] = i < p.half ? i : -1;
+      du[k] = i < p.half ? (p.halves ? i : 2 * i) : i + p.half;
+      dv[k] = i < p.half ? (p.halves ? i + p.half : 2 * i + 1) : du[k];
+      const int cu = head[k] * p.dim + du[k], cv = head[k] * p.dim + dv[k];
+      const bool is_q = head[k] < p.H;
+      const float* gw = is_q ? p.q_w : (p.k_w ? p.k_w - nq : nullptr);
+      const float rs = is_q ? rq : rk;
+      u[k] = (row[cu] + (p.bias ? p.bias[cu] : 0.f)) * rs * (gw ? gw[cu] : 1.f);
+      v[k] = (row[cv] + (p.bias ? p.bias[cv] : 0.f)) * rs * (gw ? gw[cv] : 1.f);
     }
-    const bool is_q = item < p.H;
-    const int head = is_q ? item : item - p.H, c0 = item * p.dim;
-    const float rs = is_q ? rq : rk;
-    const float* gw = is_q ? p.q_w : p.k_w;
-    if (gw) gw += (size_t)head * p.dim;
-    float* qd = p.q + ((size_t)m * p.H + head) * p.dim;
-    CT* cd = reinterpret_cast<CT*>(p.kc) + (((size_t)b * p.G + head) * p.T + (store ? t : 0)) * p.dim;
-    auto num = [&](int d) { return (row[c0 + d] + (p.bias ? p.bias[c0 + d] : 0.f)) * rs * (gw ? gw[d] : 1.f); };
-    auto put = [&](int d, float v) {
-      if (is_q) qd[d] = v;
-      else if (store) ro_st(cd + d, v);
-    };
-    // the head's pairs, then the numbers that pass
-    for (int i = lane; i < p.dim - p.half; i += 64) {
-      if (i < p.half) {
-        const int iu = p.halves ? i : 2 * i, iv = p.halves ? i + p.half : 2 * i + 1;
-        const float u = num(iu), v = num(iv);
-        put(iu, u * cs[i] - v * sn[i]);
-        put(iv, v * cs[i] + u * sn[i]);
-      } else {
-        put(i + p.half, num(i + p.half));
+#pragma unroll
+    for (int k = 0; k < QP_UNR; ++k) {
+      if (i0 + k * step >= n_qk) break;
+      float a = u[k], c = v[k];
+      if (pair[k] >= 0) {
+        const float co = cs[pair[k]], si = sn[pair[k]];
+        a = u[k] * co - v[k] * si;
+        c = v[k] * co + u[k] * si;
       }
+      if (head[k] < p.H) {
+        float* qd = p.q + (size_t)m * nq + head[k] * p.dim;
+        qd[du[k]] = a;
+        if (pair[k] >= 0) qd[dv[k]] = c;
+      } else if (store) {
+        CT* cd = reinterpret_cast<CT*>(p.kc) + (((size_t)b * p.G + (head[k] - p.H)) * p.T + t) * p.dim;
+        ro_st(cd + du[k], a);
+        if (pair[k] >= 0) ro_st(cd + dv[k], c);
+      }
+    }
+  }
+  for (int i0 = first; i0 < n_v; i0 += QP_UNR * step) {
+    float v[QP_UNR], vp[QP_UNR];
+#pragma unroll
+    for (int k = 0; k < QP_UNR; ++k) {
+      const int d = min(i0 + k * step, n_v - 1), c = nq + nk + d;
+      v[k] = row[c] + (p.bias ? p.bias[c] : 0.f);
+      vp[k] = p.v_prev ? p.v_prev[(size_t)m * n_v + d] : 0.f;
+    }
+#pragma unroll
+    for (int k = 0; k < QP_UNR; ++k) {
+      const int d = i0 + k * step;
+      if (d >= n_v) break;
+      const float x = p.v_prev ? (1.f - lam) * v[k] + lam * vp[k] : v[k];
+      if (p.v_out) p.v_out[(size_t)m * n_v + d] = x;
+      const int g = d / p.vdim;
+      if (store) ro_st(reinterpret_cast<CT*>(p.vc) + (((size_t)b * p.G + g) * p.T + t) * p.vdim + (d - g * p.vdim), x);
     }
   }
 }
@@ -162,12 +195,12 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
 int hy_qkv_prep(const QkvPrep& p, hipStream_t s) {
   if (p.B < 0 || p.S < 1 || p.H < 1 || p.G < 1 || p.H % p.G || p.dim < 1 || p.vdim < 1 || p.T < 1) return -1;
   if (p.half < 0 || 2 * p.half > p.dim || p.half > QP_MAX_HALF || (p.half > 0 && !p.freq)) return -2;
-  if (p.ld < (p.H + p.G) * p.dim + p.G * p.vdim) return -3;
+  if ((long long)(p.H + p.G) * p.dim + (long long)p.G * p.vdim > p.ld) return -3;
   if (p.v_prev && !p.lambda) return -4;
   const long long M = (long long)p.B * p.S;
   if (M == 0) return 0;
   if (M > 0x7fffffffLL) return -5;
-  const dim3 grid((unsigned)M, M <= 8 ? (unsigned)min(8, (p.H + 2 * p.G + 3) / 4) : 1u);
+  const dim3 grid((unsigned)M, M <= 8 ? (unsigned)min(8, ((p.H + p.G) * (p.dim - p.half) + 255) / 256) : 1u);
   if (p.cbf16) qkv_prep_kernel<bf16_t><<<grid, 256, 0, s>>>(p);
   else qkv_prep_kernel<float><<<grid, 256, 0, s>>>(p);
   JLA_CHECK_LAUNCH();
