@@ -501,10 +501,22 @@ template <int DK, int VT>  // dim = 16 DK, vdim = 32 VT
 __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf16_t* __restrict__ vt, int Tp) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int ql = lane & 31, hi = lane >> 5;
-  const int qblk = (gridDim.x - 1 - blockIdx.x) * 4 + wave;  // long rows first
+  // Workgroups go round the 8 XCDs by their id: where the heads divide evenly, each XCD gets whole runs of neighbouring
+  // heads (which share their keys in grouped-query attention), so that a head's keys and values pass through one L2.
+  const int nq = (p.S + 4 * AM_Q - 1) / (4 * AM_Q), heads = p.H * p.B;
+  int hb, blk;
+  if (heads % 8 == 0) {
+    const int r = blockIdx.x >> 3, hl = r / nq;
+    hb = (int)(blockIdx.x & 7) * (heads >> 3) + hl;
+    blk = r - hl * nq;
+  } else {
+    hb = blockIdx.x / nq;
+    blk = blockIdx.x - hb * nq;
+  }
+  const int qblk = (nq - 1 - blk) * 4 + wave;  // long rows first
   const int s0 = qblk * AM_Q;
   if (s0 >= p.S) return;
-  const int h = blockIdx.y, b = blockIdx.z;
+  const int b = hb / p.H, h = hb - b * p.H;
   const int g = h / (p.H / p.G);
   const int slot = *p.slot;
   const int q0 = slot + s0;                 // cache slot of this wave's first query
@@ -653,7 +665,7 @@ static int am_launch(const AttnBias& p, bf16_t* vt, int Tp, hipStream_t s) {
   attn_vt_kernel<<<dim3(Tp / 32, p.vdim / 32, p.B * p.G), 256, 0, s>>>(reinterpret_cast<const bf16_t*>(p.vc), vt, p.slot,
                                                                      p.S, p.T, Tp, p.vdim);
   JLA_CHECK_LAUNCH();
-  attn_bias_mma_kernel<DK, VT><<<dim3((p.S + 127) / 128, p.H, p.B), 256, 0, s>>>(p, vt, Tp);
+  attn_bias_mma_kernel<DK, VT><<<(unsigned)((p.S + 127) / 128 * (long long)p.H * p.B), 256, 0, s>>>(p, vt, Tp);
   JLA_CHECK_LAUNCH();
   return 0;
 }
@@ -729,7 +741,7 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
     return 0;
   }
   // (the flash kernel stores four columns at a time)
-  if (p.vt_ws && p.ldv == p.vdim && p.ldo % 4 == 0 && ((uintptr_t)p.out & (p.out_bf16 ? 7 : 15)) == 0 &&
+  if (p.vt_ws && (p.S + 127) / 128 * (long long)p.H * p.B <= 0x7fffffffLL && p.ldv == p.vdim && p.ldo % 4 == 0 && ((uintptr_t)p.out & (p.out_bf16 ? 7 : 15)) == 0 &&
       hy_attn_prefill_ws_bytes(p.B, p.S, p.G, p.dim, p.vdim, p.T, p.cbf16) > 0) {
     const int Tp = (p.T + 31) / 32 * 32;
     bf16_t* vt = reinterpret_cast<bf16_t*>(p.vt_ws);

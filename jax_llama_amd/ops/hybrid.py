@@ -1234,9 +1234,10 @@ def mlstm_prep(proj: torch.Tensor, col_i: int, col_f: int, gate_bias: torch.Tens
 
 
 # A prompt's recurrence runs as several segments side by side when one pass would leave most of the chip idle: segments
-# of at least SCAN_SEG_MIN tokens, as many as bring the launch to about SCAN_TARGET_BLOCKS workgroups.
+# of at least SCAN_SEG_MIN tokens, as many as bring the launch to SCAN_TARGET_BLOCKS workgroups (two per compute unit: a
+# count past a multiple of that leaves a partly filled last round, and segments walk the tokens twice).
 SCAN_SEG_MIN = 64
-SCAN_TARGET_BLOCKS = int(os.environ.get("JLA_HY_SCAN_BLOCKS", "1024"))
+SCAN_TARGET_BLOCKS = int(os.environ.get("JLA_HY_SCAN_BLOCKS", "512"))
 
 
 def _scan_segments(b: int, s: int, heads: int, dim: int, cols: int, device):

@@ -427,8 +427,8 @@ def _run_rec(w, mc, h, eps, device, portions, dtype=F32):
 
 
 @pytest.mark.parametrize("device", DEVICES)
-@pytest.mark.parametrize("heads,dim,vdim,t", [(3, 12, 20, 70), (1, 1, 1, 9), (2, 64, 64, 300), (5, 17, 33, 150), (1, 130, 9, 140),
-                                              (9, 16, 257, 40), (1, 600, 4, 130)])
+@pytest.mark.parametrize("heads,dim,vdim,t", [(3, 12, 20, 70), (1, 1, 1, 9), (2, 64, 64, 300), (5, 17, 33, 200), (1, 130, 9, 260),
+                                              (9, 16, 257, 40), (1, 600, 4, 210)])
 def test_running_memory_mechanism(device, heads, dim, vdim, t):
     """The recurrence against the oracle, output and carried state: one pass, segments side by side (128 tokens and more),
     portions with single tokens and pairs, token by token."""
@@ -441,6 +441,23 @@ def test_running_memory_mechanism(device, heads, dim, vdim, t):
     for portions in ([t], [1] * t, [2, 1, t - 6, 3]):
         got, st = _run_rec(w, mc, h, eps, device, portions)
         assert err(got, ref) < 2e-5 and err(st, state) < 2e-5, portions
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("seg_min", [4, 16])
+def test_running_memory_in_short_segments(seg_min, monkeypatch):
+    """Many short segments side by side, an uneven last one, a second portion that starts from a carried state."""
+    monkeypatch.setattr(hy, "SCAN_SEG_MIN", seg_min)
+    t, d, eps = 75, 40, 1e-6
+    g = torch.Generator().manual_seed(11)
+    h = torch.randn(t, d, generator=g)
+    for mc in (_rec(3, 8, 12), _rec(2, 40, 33), _rec(1, 130, 4)):
+        w = _rec_weights(g, mc, d)
+        ref, state = of.hgrn2(w, "m.", mc, h.double().numpy(), eps, return_state=True)
+        for portions in ([75], [40, 35], [9, 66]):
+            assert hy._scan_segments(1, portions[-1], mc["heads"], mc["dim"], mc["vdim"], "cuda")[0] > 1
+            got, st = _run_rec(w, mc, h, eps, "cuda", portions)
+            assert err(got, ref) < 2e-5 and err(st, state) < 2e-5, (mc, portions)
 
 
 @pytest.mark.parametrize("device", DEVICES)
