@@ -1065,3 +1065,220 @@ class FokisunConfig:
 
     def __repr__(self) -> str:
         return f"FokisunConfig {json.dumps(self.to_dict(), sort_keys=True)}"
+
+
+# -------------------------------------------------------------------------------------
+# Zopupel: differential attention and attention whose values are its keys, biased softmax routing, norms on both sides of
+# every sublayer
+# -------------------------------------------------------------------------------------
+@dataclass
+class RotarySpec:
+    """Rotary positions on the first ``dims`` numbers of a head (base ``base``). ``factor``: frequencies divided by it, or,
+    with ``original`` > 0 (the context length the base was made for), divided only for the pairs that turn slowly: a ramp
+    between the pairs of ``fast`` and ``slow`` full turns over ``original`` positions, and a factor on cosine and sine."""
+
+    base: float
+    dims: int
+    factor: float = 1.0
+    original: float = 0.0
+    fast: float = 32.0
+    slow: float = 1.0
+
+    @classmethod
+    def from_dict(cls, d: Optional[Dict[str, Any]], dim: int) -> Optional["RotarySpec"]:
+        if not d or not int(d.get("dims", dim)):
+            return None
+        sc = d.get("scaling") or {}
+        out = cls(base=float(d["base"]), dims=int(d.get("dims", dim)), factor=float(sc.get("factor", 1.0)),
+                  original=float(sc.get("original", 0) or 0), fast=float(sc.get("fast", 32.0)),
+                  slow=float(sc.get("slow", 1.0)))
+        if out.dims % 2 or not 0 < out.dims <= dim:
+            raise ValueError(f"rot.dims {out.dims} must be even and at most the head's {dim}")
+        if not out.factor > 0.0 or out.original < 0.0 or not (out.fast > 0.0 and out.slow > 0.0) or \
+                (out.original and not (out.base > 0.0 and out.base != 1.0)):
+            raise ValueError("rot.scaling: factor, fast and slow must be positive")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        out: Dict[str, Any] = {"base": self.base, "dims": self.dims}
+        if self.original:
+            out["scaling"] = {"factor": self.factor, "original": self.original, "fast": self.fast, "slow": self.slow}
+        elif self.factor != 1.0:
+            out["scaling"] = {"factor": self.factor}
+        return out
+
+    def freqs(self, device):
+        """``(float64 [dims / 2] turn per position of every pair, factor on cosine and sine)``."""
+        from .ops import hybrid as hy
+        if self.original:
+            return hy.yarn_freqs(self.base, self.dims, self.factor, self.original, self.fast, self.slow, device)
+        return hy.rotary_freqs(self.base, self.dims, device) / self.factor, 1.0
+
+
+@dataclass
+class DifferentialAttentionSpec:
+    """Differential attention: ``heads`` query heads over ``kv_heads`` key / value heads, two maps of ``dim`` numbers per q / k
+    head, values of ``vdim``; ``diff`` the constant part of the second map's weight. ``kv_from``: the layer has no keys and
+    values of its own and reads that layer's."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    rot: Optional[RotarySpec] = None
+    kv_from: Optional[int] = None
+    type = "attention"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "DifferentialAttentionSpec":
+        heads, dim = int(d["heads"]), int(d["dim"])
+        out = cls(heads=heads, kv_heads=int(d.get("kv_heads", heads)), dim=dim, vdim=int(d.get("vdim", dim)),
+                  scale=float(d["scale"]), diff=float(d["diff"]), rot=RotarySpec.from_dict(d.get("rot"), dim),
+                  kv_from=int(d["kv_from"]) if d.get("kv_from") is not None else None)
+        if out.heads % out.kv_heads:
+            raise ValueError("heads must be divisible by kv_heads")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        out: Dict[str, Any] = dict(heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, scale=self.scale,
+                                   diff=self.diff)
+        if self.rot:
+            out["rot"] = self.rot.to_dict()
+        if self.kv_from is not None:
+            out["kv_from"] = self.kv_from
+        return out
+
+
+@dataclass
+class KeyValueAttentionSpec:
+    """Softmax attention whose values are the keys as projected: biases, q and k normed over their whole projections, rotary
+    positions, one added to the softmax denominator."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    rot: Optional[RotarySpec] = None
+    type = "attention_2"
+    window = 0
+
+    @property
+    def vdim(self) -> int:
+        return self.dim
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "KeyValueAttentionSpec":
+        heads, dim = int(d["heads"]), int(d["dim"])
+        out = cls(heads=heads, kv_heads=int(d.get("kv_heads", heads)), dim=dim, scale=float(d["scale"]),
+                  rot=RotarySpec.from_dict(d.get("rot"), dim))
+        if out.heads % out.kv_heads:
+            raise ValueError("heads must be divisible by kv_heads")
+        if int(d.get("vdim", dim)) != dim:
+            raise ValueError("values that are the keys have their size: vdim must equal dim")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        out: Dict[str, Any] = dict(heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, scale=self.scale)
+        if self.rot:
+            out["rot"] = self.rot.to_dict()
+        return out
+
+
+@dataclass
+class SharedExpertMoESpec:
+    """Softmax-routed mixture of ``experts`` gated experts of width ``ff``, ``top`` of them per token (weights over the chosen
+    logits); an optional shared expert of width ``shared_ff``."""
+
+    experts: int
+    top: int
+    ff: int
+    shared_ff: int = 0
+    kind = "moe"
+
+    @classmethod
+    def from_dict(cls, d: Optional[Dict[str, Any]]) -> Optional["SharedExpertMoESpec"]:
+        if d is None:
+            return None
+        if d.get("kind", "moe") != "moe":
+            raise ValueError(f"unknown feed-forward kind {d.get('kind')!r}")
+        out = cls(experts=int(d["router"]["experts"]), top=int(d["router"]["top"]), ff=int(d["expert"]["ff"]),
+                  shared_ff=int((d.get("shared") or {}).get("ff", 0)))
+        if not 1 <= out.top <= out.experts:
+            raise ValueError(f"router: top {out.top} of {out.experts} experts")
+        return out
+
+    def to_dict(self) -> Dict[str, Any]:
+        out: Dict[str, Any] = {"kind": "moe", "expert": {"ff": self.ff},
+                               "router": {"experts": self.experts, "top": self.top}}
+        if self.shared_ff:
+            out["shared"] = {"ff": self.shared_ff}
+        return out
+
+
+class ZopupelConfig:
+    """Zopupel decoder: ``config.json`` with ``architecture: "Zopupel"``, ``vocab``, ``width``, ``norm.eps``,
+    ``residual_mult`` and a ``layers`` list of ``{type, mixer, mlp}`` entries; ``type`` is ``attention`` (differential) or
+    ``attention_2``, ``mlp`` null or a ``SharedExpertMoESpec`` entry."""
+
+    model_type = "zopupel"
+    architecture = "Zopupel"
+    MIXERS = {"attention": DifferentialAttentionSpec, "attention_2": KeyValueAttentionSpec}
+
+    def __init__(self, vocab_size: int, hidden_size: int, layers, norm_eps: float = 1e-6, residual_mult: float = 1.0,
+                 pad_token_id: int = -1, eos_token_id: Optional[int] = None):
+        self.vocab_size = int(vocab_size)
+        self.hidden_size = int(hidden_size)
+        self.layers = list(layers)
+        self.norm_eps = float(norm_eps)
+        self.residual_mult = float(residual_mult)
+        self.pad_token_id = pad_token_id
+        self.eos_token_id = eos_token_id
+        for i, ls in enumerate(self.layers):
+            j = getattr(ls.mixer, "kv_from", None)
+            if j is not None:
+                src = self.layers[j].mixer if 0 <= j < i else None
+                if not isinstance(src, DifferentialAttentionSpec) or src.kv_from is not None:
+                    raise ValueError(f"layer {i}: kv_from {j} is not an earlier attention layer with its own keys")
+                if (src.kv_heads, src.dim, src.vdim) != (ls.mixer.kv_heads, ls.mixer.dim, ls.mixer.vdim):
+                    raise ValueError(f"layer {i}: key / value geometry differs from layer {j}'s")
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "ZopupelConfig":
+        layers = []
+        for i, e in enumerate(d["layers"]):
+            if e["type"] not in cls.MIXERS:
+                raise ValueError(f"layer {i}: Zopupel has no mixer {e['type']!r}")
+            layers.append(LayerSpec(cls.MIXERS[e["type"]].from_dict(e["mixer"]), SharedExpertMoESpec.from_dict(e.get("mlp"))))
+        return cls(vocab_size=d["vocab"], hidden_size=d["width"], layers=layers, norm_eps=d["norm"]["eps"],
+                   residual_mult=d.get("residual_mult", 1.0), pad_token_id=d.get("pad_token_id", -1),
+                   eos_token_id=d.get("eos_token_id"))
+
+    def to_dict(self) -> Dict[str, Any]:
+        return {"architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size,
+                "norm": {"eps": self.norm_eps}, "residual_mult": self.residual_mult,
+                "layers": [{"type": ls.mixer.type, "mixer": ls.mixer.to_dict(),
+                            "mlp": ls.mlp.to_dict() if ls.mlp is not None else None} for ls in self.layers]}
+
+    def save_pretrained(self, save_directory: str) -> None:
+        os.makedirs(save_directory, exist_ok=True)
+        with open(os.path.join(save_directory, "config.json"), "w") as f:
+            json.dump(self.to_dict(), f, indent=1, sort_keys=True)
+
+    @classmethod
+    def from_pretrained(cls, path: str) -> "ZopupelConfig":
+        if os.path.isdir(path):
+            path = os.path.join(path, "config.json")
+        with open(path) as f:
+            return cls.from_dict(json.load(f))
+
+    def __eq__(self, other: object) -> bool:
+        return isinstance(other, ZopupelConfig) and self.to_dict() == other.to_dict()
+
+    def __repr__(self) -> str:
+        return f"ZopupelConfig {json.dumps(self.to_dict(), sort_keys=True)}"

@@ -21,6 +21,12 @@
 // projection columns) multiplies the normalised output in the kernels that write it; the output may be a column slice of
 // a wider row, in fp32 or bf16. Values may be the leading columns of wider rows (ldv): a latent cache whose rows carry a
 // rotated key part behind the latent serves as keys (whole row) and values (latent).
+// Differential heads (maps = 2): an output head has two query / key maps over the same values; each map is a softmax of its
+// own, and the head's output is RMS-normed (a1 - lambda a2) times a constant. A key row holds both maps side by side (ldk =
+// 2 dim). Scores are counted per map: query head 2 h + b is map b of head h, and per-head score parameters (sink, factor,
+// bias column) are indexed by it. Prefill: one wave runs both maps of its query (plain), or a pair of waves runs one map
+// each over the same 32 queries and joins them through LDS (MFMA). Decode: the splits of both maps side by side, joined by
+// the merge.
 #include "hy_util.h"
 #include "hybrid.h"
 
@@ -106,6 +112,14 @@ JLA_DEV AbSpan ab_span(const AttnBias& p, int qi) {
   sp.n = sp.kf + qi + 1 - sp.lo;
   return sp;
 }
+// query head vh = map vh % maps of output head vh / maps: its key / value head, and its keys' offset within a key row
+struct AbMap {
+  int g, koff;
+};
+JLA_DEV AbMap ab_map(const AttnBias& p, int vh) {
+  const int h = vh / p.maps;
+  return {h / (p.H / p.G), (vh - h * p.maps) * p.dim};
+}
 JLA_DEV int ab_key(const AbSpan& sp, int v) { return v < sp.kf ? v : sp.lo + (v - sp.kf); }
 // gate of column c of head h: one per head, or one per column
 JLA_DEV float ab_gate(const AttnBias& p, size_t m, int h, int c) {
@@ -117,17 +131,17 @@ JLA_DEV void ab_out(const AttnBias& p, size_t m, int h, int c, float v) {
   else reinterpret_cast<float*>(p.out)[at] = v;
 }
 
-// One wave: visible keys number [j_lo, j_hi) of query (b, h) at slot qi (span); returns the running max m, sum l and
+// One wave: visible keys number [j_lo, j_hi) of query (b, query head h) at slot qi (span); returns the running max m, sum l and
 // unnormalised acc. with_sink: the wave whose keys start the row also counts the head's sink.
 template <typename CT, int VREG>  // VREG: value columns per lane (vdim <= 64 VREG)
 JLA_DEV void ab_wave(const AttnBias& p, const float* qs, int b, int h, int qi, const AbSpan& span, int j_lo, int j_hi,
                      bool with_sink, float& m_run, float& l_run, float* acc) {
   constexpr int KB = VREG <= 2 ? 16 : 8;  // keys whose value rows are in flight at a time
   const int lane = threadIdx.x & 63;
-  const int g = h / (p.H / p.G);
-  const CT* kbase = reinterpret_cast<const CT*>(p.kc) + ((size_t)b * p.G + g) * p.T * p.dim;
-  const CT* vbase = reinterpret_cast<const CT*>(p.vc) + ((size_t)b * p.G + g) * p.T * p.ldv;
-  const bool fastk = (p.dim & 7) == 0 && ((uintptr_t)kbase & 15) == 0;
+  const AbMap mp = ab_map(p, h);
+  const CT* kbase = reinterpret_cast<const CT*>(p.kc) + ((size_t)b * p.G + mp.g) * p.T * p.ldk + mp.koff;
+  const CT* vbase = reinterpret_cast<const CT*>(p.vc) + ((size_t)b * p.G + mp.g) * p.T * p.ldv;
+  const bool fastk = ((p.dim | p.ldk) & 7) == 0 && ((uintptr_t)kbase & 15) == 0;
   const bool sunk = with_sink && p.sink;
   const float hs = p.head_scale ? p.head_scale[h] : 1.f;
   m_run = sunk ? p.sink[h] : -INFINITY;
@@ -139,7 +153,7 @@ JLA_DEV void ab_wave(const AttnBias& p, const float* qs, int b, int h, int qi, c
     const int kj = ab_key(span, min(j, j_hi - 1));  // cache slot of this lane's key
     float sc = -INFINITY;
     if (j < j_hi) {
-      const CT* kr = kbase + (size_t)kj * p.dim;
+      const CT* kr = kbase + (size_t)kj * p.ldk;
       float d0 = 0.f, d1 = 0.f;
       if (fastk) {  // whole 16-byte groups: branch-free loads the scheduler can batch
 #pragma unroll 4
@@ -157,7 +171,7 @@ JLA_DEV void ab_wave(const AttnBias& p, const float* qs, int b, int h, int qi, c
       }
       sc = (d0 + d1) * p.scale * hs;
       if (p.softcap > 0.f) sc = p.softcap * tanhf(sc / p.softcap);
-      if (p.bias) sc += p.bias[(size_t)min(qi - kj, p.nbias - 1) * p.H + h];
+      if (p.bias) sc += p.bias[(size_t)min(qi - kj, p.nbias - 1) * (p.H * p.maps) + h];
     }
     const float m_new = fmaxf(m_run, wave_max(sc));
     const float corr = expf(m_run - m_new);  // first chunk: exp(-inf) = 0
@@ -196,6 +210,43 @@ JLA_DEV void ab_split_range(const AttnBias& p, const AbSpan& span, int sp, int& 
   j_hi = min(n, j_lo + per);
 }
 
+// prefill of differential heads: grid (ceil(S / 4), H, B), one wave per query, its two maps one after the other
+template <typename CT, int VREG>
+__global__ void __launch_bounds__(256) attn_diff_prefill_kernel(AttnBias p) {
+  __shared__ float qs_all[4][AB_MAX_DIM];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int s = blockIdx.x * 4 + wave, h = blockIdx.y, b = blockIdx.z;
+  if (s >= p.S) return;
+  float* qs = qs_all[wave];
+  const size_t m = (size_t)b * p.S + s;
+  const int qi = min(*p.slot + s, p.T - 1);
+  const AbSpan span = ab_span(p, qi);
+  float o[VREG];
+#pragma unroll
+  for (int i = 0; i < VREG; ++i) o[i] = 0.f;
+  for (int map = 0; map < 2; ++map) {
+    const float* q = p.q + (m * p.H * 2 + 2 * h + map) * p.dim;
+    __builtin_amdgcn_wave_barrier();
+    for (int d = lane; d < p.dim; d += 64) qs[d] = q[d];
+    __builtin_amdgcn_wave_barrier();
+    float m_run, l_run, acc[VREG];
+    ab_wave<CT, VREG>(p, qs, b, 2 * h + map, qi, span, 0, span.n, true, m_run, l_run, acc);
+    const float w = (map ? -p.diff_lambda : 1.f) / l_run;
+#pragma unroll
+    for (int i = 0; i < VREG; ++i) o[i] = fmaf(w, acc[i], o[i]);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VREG; ++i)
+    if (lane + 64 * i < p.vdim) ss = fmaf(o[i], o[i], ss);
+  const float sc = p.diff_gain / sqrtf(wave_sum(ss) / (float)p.vdim + p.diff_eps);
+#pragma unroll
+  for (int i = 0; i < VREG; ++i) {
+    const int c = lane + 64 * i;
+    if (c < p.vdim) ab_out(p, m, h, c, o[i] * (sc * ab_gate(p, m, h, c)));
+  }
+}
+
 // prefill: grid (ceil(S / 4), H, B), one wave per query
 template <typename CT, int VREG>
 __global__ void __launch_bounds__(256) attn_bias_prefill_kernel(AttnBias p) {
@@ -220,13 +271,14 @@ __global__ void __launch_bounds__(256) attn_bias_prefill_kernel(AttnBias p) {
   }
 }
 
-// decode: grid (splits, H, B), one wave per (row, head, split); partial = [m, l, acc[vdim]]
+// decode: grid (splits, H maps, B), one wave per (row, query head, split); partial = [m, l, acc[vdim]]
 template <typename CT, int VREG>
 __global__ void __launch_bounds__(64) attn_bias_decode_kernel(AttnBias p) {
   __shared__ float qs[AB_MAX_DIM];
   const int lane = threadIdx.x;
   const int sp = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
-  const float* q = p.q + ((size_t)b * p.H + h) * p.dim;
+  const int heads = p.H * p.maps;
+  const float* q = p.q + ((size_t)b * heads + h) * p.dim;
   for (int d = lane; d < p.dim; d += 64) qs[d] = q[d];
   __syncthreads();
   const int qi = min(*p.slot, p.T - 1);
@@ -235,7 +287,7 @@ __global__ void __launch_bounds__(64) attn_bias_decode_kernel(AttnBias p) {
   ab_split_range(p, span, sp, j_lo, j_hi);
   float m_run, l_run, acc[VREG];
   ab_wave<CT, VREG>(p, qs, b, h, qi, span, j_lo, j_hi, sp == 0, m_run, l_run, acc);
-  float* w = p.ws + (((size_t)b * p.H + h) * p.splits + sp) * (p.vdim + 2);
+  float* w = p.ws + (((size_t)b * heads + h) * p.splits + sp) * (p.vdim + 2);
   if (lane == 0) {
     w[0] = m_run;
     w[1] = l_run;
@@ -256,8 +308,9 @@ __global__ void __launch_bounds__(64) attn_bias_decode_fast_kernel(AttnBias p) {
   __shared__ float qs[dim];
   const int lane = threadIdx.x;
   const int sp = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
-  const int g = h / (p.H / p.G);
-  const float* q = p.q + ((size_t)b * p.H + h) * dim;
+  const AbMap mp = ab_map(p, h);
+  const int heads = p.H * p.maps;
+  const float* q = p.q + ((size_t)b * heads + h) * dim;
   float qv[dim / 64];
 #pragma unroll
   for (int i = 0; i < dim / 64; ++i) qv[i] = q[lane + 64 * i];
@@ -265,8 +318,8 @@ __global__ void __launch_bounds__(64) attn_bias_decode_fast_kernel(AttnBias p) {
   int j_lo, j_hi;
   const AbSpan span = ab_span(p, qi);
   ab_split_range(p, span, sp, j_lo, j_hi);
-  const bf16_t* kbase = reinterpret_cast<const bf16_t*>(p.kc) + ((size_t)b * p.G + g) * p.T * dim;
-  const bf16_t* vbase = reinterpret_cast<const bf16_t*>(p.vc) + ((size_t)b * p.G + g) * p.T * p.ldv;
+  const bf16_t* kbase = reinterpret_cast<const bf16_t*>(p.kc) + ((size_t)b * p.G + mp.g) * p.T * p.ldk + mp.koff;
+  const bf16_t* vbase = reinterpret_cast<const bf16_t*>(p.vc) + ((size_t)b * p.G + mp.g) * p.T * p.ldv;
   const bool sunk = p.sink && sp == 0;
   const float hs = p.head_scale ? p.head_scale[h] : 1.f;
   float m_run = sunk ? p.sink[h] : -INFINITY, l_run = sunk ? 1.f : 0.f, acc[VREG];
@@ -277,8 +330,8 @@ __global__ void __launch_bounds__(64) attn_bias_decode_fast_kernel(AttnBias p) {
     const int j = j0 + lane, jc = ab_key(span, min(j, j_hi - 1));  // (jc: the cache slot)
     u32x4 kf[DK8];
 #pragma unroll
-    for (int u = 0; u < DK8; ++u) kf[u] = *reinterpret_cast<const u32x4*>(kbase + (size_t)jc * dim + 8 * u);
-    const float bl = p.bias ? p.bias[(size_t)min(qi - jc, p.nbias - 1) * p.H + h] : 0.f;
+    for (int u = 0; u < DK8; ++u) kf[u] = *reinterpret_cast<const u32x4*>(kbase + (size_t)jc * p.ldk + 8 * u);
+    const float bl = p.bias ? p.bias[(size_t)min(qi - jc, p.nbias - 1) * heads + h] : 0.f;
     bf16_t vv[64][VREG];
 #pragma unroll
     for (int jj = 0; jj < 64; ++jj) {
@@ -321,7 +374,7 @@ __global__ void __launch_bounds__(64) attn_bias_decode_fast_kernel(AttnBias p) {
       for (int i = 0; i < VREG; ++i) acc[i] = fmaf(pj, bf2f(vv[jj][i]), acc[i]);
     }
   }
-  float* w = p.ws + (((size_t)b * p.H + h) * p.splits + sp) * (vdim + 2);
+  float* w = p.ws + (((size_t)b * heads + h) * p.splits + sp) * (vdim + 2);
   if (lane == 0) {
     w[0] = m_run;
     w[1] = l_run;
@@ -462,6 +515,45 @@ __global__ void __launch_bounds__(64) attn_bias_merge_kernel(AttnBias p) {
   if (c0 + lane < p.vdim) ab_out(p, b, h, c, a / l * gt);
 }
 
+// differential heads: grid (H, B), a wave per 64 value columns; both maps' splits merged, then the head's norm over all of
+// its columns
+__global__ void __launch_bounds__(64 * AB_MAX_VREG) attn_diff_merge_kernel(AttnBias p) {
+  __shared__ float red[AB_MAX_VREG];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.x, b = blockIdx.y, waves = blockDim.x >> 6;
+  const int c = min((int)threadIdx.x, p.vdim - 1);
+  float o = 0.f;
+#pragma unroll
+  for (int map = 0; map < 2; ++map) {
+    const float* w = p.ws + (((size_t)b * p.H + h) * 2 + map) * p.splits * (p.vdim + 2);
+    float ms = -INFINITY, ls = 0.f;
+    if (lane < p.splits) {
+      ms = w[(size_t)lane * (p.vdim + 2)];
+      ls = w[(size_t)lane * (p.vdim + 2) + 1];
+    }
+    float part[64];
+#pragma unroll
+    for (int sp = 0; sp < 64; ++sp) part[sp] = w[(size_t)min(sp, p.splits - 1) * (p.vdim + 2) + 2 + c];
+    const float m = wave_max(ls > 0.f ? ms : -INFINITY);
+    const float wt = ls > 0.f ? expf(ms - m) : 0.f;
+    const float l = wave_sum(ls * wt);
+    float a = 0.f;
+#pragma unroll
+    for (int sp = 0; sp < 64; ++sp) {
+      const float ws = __shfl(wt, sp, 64);
+      a = fmaf(part[sp], sp < p.splits ? ws : 0.f, a);
+    }
+    o = fmaf(map ? -p.diff_lambda : 1.f, a / l, o);
+  }
+  const bool on = (int)threadIdx.x < p.vdim;
+  float ss = wave_sum(on ? o * o : 0.f);
+  if (lane == 0) red[wave] = ss;
+  __syncthreads();
+  ss = 0.f;
+  for (int i = 0; i < waves; ++i) ss += red[i];
+  const float sc = p.diff_gain / sqrtf(ss / (float)p.vdim + p.diff_eps);
+  if (on) ab_out(p, b, h, c, o * sc * ab_gate(p, b, h, c));
+}
+
 // ---- MFMA flash prefill (bf16 caches) ----------------------------------------------------------------------------------
 // One wave = 32 queries of one head, no LDS and no barriers. Keys go by in tiles of 32:
 //   S^T = K Q^T on v_mfma_f32_32x32x16_bf16 with the QUERY on the lane (lane l: query l & 31; its 16 accumulators are 16
@@ -497,13 +589,18 @@ JLA_DEV float am_tanh(float x) {  // 1 - 2 / (e^(2x) + 1), saturating cleanly fo
   return 1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f);
 }
 
-template <int DK, int VT>  // dim = 16 DK, vdim = 32 VT
+// MAPS = 2 (differential heads): waves 2 t and 2 t + 1 of a workgroup run the two maps of query tile t; the second hands its
+// normalised output to the first through LDS, which subtracts, norms and stores.
+template <int DK, int VT, int MAPS>  // dim = 16 DK, vdim = 32 VT
 __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf16_t* __restrict__ vt, int Tp) {
+  constexpr int TILES = 4 / MAPS;  // query tiles per workgroup
+  __shared__ float joined[MAPS == 2 ? TILES * VT * 16 * 64 : 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int map = wave % MAPS;
   const int ql = lane & 31, hi = lane >> 5;
   // Workgroups go round the 8 XCDs by their id: where the heads divide evenly, each XCD gets whole runs of neighbouring
   // heads (which share their keys in grouped-query attention), so that a head's keys and values pass through one L2.
-  const int nq = (p.S + 4 * AM_Q - 1) / (4 * AM_Q), heads = p.H * p.B;
+  const int nq = (p.S + TILES * AM_Q - 1) / (TILES * AM_Q), heads = p.H * p.B;
   int hb, blk;
   if (heads % 8 == 0) {
     const int r = blockIdx.x >> 3, hl = r / nq;
@@ -513,11 +610,12 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
     hb = blockIdx.x / nq;
     blk = blockIdx.x - hb * nq;
   }
-  const int qblk = (nq - 1 - blk) * 4 + wave;  // long rows first
+  const int qblk = (nq - 1 - blk) * TILES + wave / MAPS;  // long rows first
   const int s0 = qblk * AM_Q;
-  if (s0 >= p.S) return;
+  const bool live = s0 < p.S;
+  if (MAPS == 1 && !live) return;  // (a pair of waves without queries stays for the workgroup's barrier)
   const int b = hb / p.H, h = hb - b * p.H;
-  const int g = h / (p.H / p.G);
+  const int g = h / (p.H / p.G), vh = h * MAPS + map;
   const int slot = *p.slot;
   const int q0 = slot + s0;                 // cache slot of this wave's first query
   const int sq = min(s0 + ql, p.S - 1);     // (surplus lanes repeat the last query; never stored)
@@ -526,7 +624,7 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
   // Q as the B operand: query ql, k-slots 16 kk + 8 hi + e
   bf16x8_t qf[DK];
   {
-    const float* q = p.q + (((size_t)b * p.S + sq) * p.H + h) * dim + 8 * hi;
+    const float* q = p.q + (((size_t)b * p.S + sq) * (p.H * MAPS) + vh) * dim + 8 * hi;
 #pragma unroll
     for (int kk = 0; kk < DK; ++kk) {
       float f[8];
@@ -534,7 +632,7 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
       qf[kk] = __builtin_bit_cast(bf16x8_t, pack8(f));
     }
   }
-  const bf16_t* kbase = reinterpret_cast<const bf16_t*>(p.kc) + ((size_t)b * p.G + g) * p.T * dim;
+  const bf16_t* kbase = reinterpret_cast<const bf16_t*>(p.kc) + ((size_t)b * p.G + g) * p.T * p.ldk + map * dim;
   const bf16_t* vbase = vt + ((size_t)b * p.G + g) * vdim * Tp;
   const int krow = (ql & 0x13) | ((ql & 4) << 1) | ((ql & 8) >> 1);  // bits 2 and 3 swapped
   f32x16 o[VT];
@@ -543,10 +641,10 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[v][r] = 0.f;
   // (l_run holds this half-wave's part of the sum: the sink counts once, in the lower half)
-  float m_run = p.sink ? p.sink[h] : -INFINITY, l_run = p.sink && hi == 0 ? 1.f : 0.f;
-  const int q_last = min(q0 + AM_Q - 1, slot + p.S - 1);
+  float m_run = p.sink ? p.sink[vh] : -INFINITY, l_run = p.sink && hi == 0 ? 1.f : 0.f;
+  const int q_last = live ? min(q0 + AM_Q - 1, slot + p.S - 1) : -1;  // (no tile is walked without queries)
   const float inv_cap = p.softcap > 0.f ? 1.f / p.softcap : 0.f;
-  const float hs = p.head_scale ? p.head_scale[h] : 1.f;
+  const float hs = p.head_scale ? p.head_scale[vh] : 1.f;
   // block-local mask: this query's first key, the last query's (the largest of the wave), and the tile the walk starts at
   const int lo_q = ab_span(p, qi).lo, lo_last = ab_span(p, q_last).lo;
   const int j_begin = ab_span(p, q0).lo / AM_K * AM_K;
@@ -558,7 +656,7 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
   // batch: nothing else hides the loads)
   u32x4 kn[DK], vn[2][VT];
   auto fetch = [&](int j0) {
-    const bf16_t* kr = kbase + (size_t)min(j0 + krow, p.T - 1) * dim + 8 * hi;
+    const bf16_t* kr = kbase + (size_t)min(j0 + krow, p.T - 1) * p.ldk + 8 * hi;
 #pragma unroll
     for (int kk = 0; kk < DK; ++kk) kn[kk] = *reinterpret_cast<const u32x4*>(kr + 16 * kk);
 #pragma unroll
@@ -589,7 +687,7 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
     float bl = 0.f;
     const int dbase = q0 - j0 - (AM_K - 1);
     const bool far = p.bias && dbase >= p.nbias - 1;
-    if (p.bias) bl = p.bias[(size_t)min(max(dbase + lane, 0), p.nbias - 1) * p.H + h];
+    if (p.bias) bl = p.bias[(size_t)min(max(dbase + lane, 0), p.nbias - 1) * (p.H * MAPS) + vh];
     // some (query, key) of the tile is masked
     const bool diag = j0 + AM_K - 1 > q0 || (j0 < lo_last && j0 + AM_K - 1 >= kfirst);
     float tmax = -INFINITY;
@@ -639,9 +737,31 @@ __global__ void __launch_bounds__(256) attn_bias_mma_kernel(AttnBias p, const bf
     }
   }
   l_run += __shfl_xor(l_run, 32, 64);
-  if (s0 + ql >= p.S) return;
   const size_t m = (size_t)b * p.S + s0 + ql;
-  const float inv = p.gate && !p.gate_cols ? ab_gate(p, m, h, 0) / l_run : 1.f / l_run;
+  float inv = 1.f / l_run;
+  if constexpr (MAPS == 2) {
+    float* mine = joined + (wave / MAPS) * VT * 16 * 64 + lane;
+    if (map == 1) {
+#pragma unroll
+      for (int v = 0; v < VT; ++v)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) mine[(v * 16 + r) * 64] = o[v][r] * inv;
+    }
+    __syncthreads();
+    if (map == 1) return;
+    float ss = 0.f;  // (a query's columns: this lane's and those of lane ^ 32)
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        o[v][r] = o[v][r] * inv - p.diff_lambda * mine[(v * 16 + r) * 64];
+        ss = fmaf(o[v][r], o[v][r], ss);
+      }
+    ss += __shfl_xor(ss, 32, 64);
+    inv = p.diff_gain / sqrtf(ss / (float)vdim + p.diff_eps);
+  }
+  if (s0 + ql >= p.S) return;
+  if (p.gate && !p.gate_cols) inv *= ab_gate(p, m, h, 0);
   const size_t at = m * p.ldo + (size_t)h * vdim;
   const float* gt = p.gate && p.gate_cols ? p.gate + m * p.ldg + (size_t)h * vdim : nullptr;
 #pragma unroll
@@ -665,7 +785,9 @@ static int am_launch(const AttnBias& p, bf16_t* vt, int Tp, hipStream_t s) {
   attn_vt_kernel<<<dim3(Tp / 32, p.vdim / 32, p.B * p.G), 256, 0, s>>>(reinterpret_cast<const bf16_t*>(p.vc), vt, p.slot,
                                                                      p.S, p.T, Tp, p.vdim);
   JLA_CHECK_LAUNCH();
-  attn_bias_mma_kernel<DK, VT><<<(unsigned)((p.S + 127) / 128 * (long long)p.H * p.B), 256, 0, s>>>(p, vt, Tp);
+  const long long hb = (long long)p.H * p.B;
+  if (p.maps == 2) attn_bias_mma_kernel<DK, VT, 2><<<(unsigned)((p.S + 63) / 64 * hb), 256, 0, s>>>(p, vt, Tp);
+  else attn_bias_mma_kernel<DK, VT, 1><<<(unsigned)((p.S + 127) / 128 * hb), 256, 0, s>>>(p, vt, Tp);
   JLA_CHECK_LAUNCH();
   return 0;
 }
@@ -716,19 +838,22 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
   if (p.dim < 1 || p.dim > AB_MAX_DIM || p.vdim < 1 || p.vdim > 64 * AB_MAX_VREG) return -2;
   if (p.bias && p.nbias < 1) return -3;
   if (p.chunk < 0 || p.window < 0 || p.keep_first < 0 || (p.chunk > 0 && p.window > 0)) return -7;
+  if (p.maps != 1 && p.maps != 2) return -10;
+  if (p.ldk < p.maps * p.dim) return -8;
   if (p.ldv < p.vdim || (p.gate && p.ldg < (p.gate_cols ? p.H * p.vdim : p.H)) || p.ldo < p.H * p.vdim) return -8;
   if (p.B == 0) return 0;
-  if (p.H > 65535 || p.B > 65535) return -4;
+  if ((long long)p.H * p.maps > 65535 || p.B > 65535) return -4;
   if (p.S == 1) {
     if (p.splits < 1 || !p.ws) return -5;
     if (p.splits > 64) return -6;  // (the merge holds one split per lane)
-    dim3 grid(p.splits, p.H, p.B);
-    if (p.cbf16 && (p.dim == 64 || p.dim == 128) && (p.vdim == 64 || p.vdim == 128) && p.ldv == p.vdim) {
+    dim3 grid(p.splits, p.H * p.maps, p.B);
+    if (p.cbf16 && (p.dim == 64 || p.dim == 128) && (p.vdim == 64 || p.vdim == 128) && p.ldv == p.vdim && p.ldk % 8 == 0 &&
+        ((uintptr_t)p.kc & 15) == 0) {
       if (p.dim == 64 && p.vdim == 64) attn_bias_decode_fast_kernel<8, 1><<<grid, 64, 0, s>>>(p);
       else if (p.dim == 64) attn_bias_decode_fast_kernel<8, 2><<<grid, 64, 0, s>>>(p);
       else if (p.vdim == 64) attn_bias_decode_fast_kernel<16, 1><<<grid, 64, 0, s>>>(p);
       else attn_bias_decode_fast_kernel<16, 2><<<grid, 64, 0, s>>>(p);
-    } else if (p.cbf16 && p.kc == p.vc && p.G == 1 && p.ldv == p.dim && p.vdim <= p.dim && p.vdim % 8 == 0 &&
+    } else if (p.cbf16 && p.maps == 1 && p.kc == p.vc && p.G == 1 && p.ldk == p.dim && p.ldv == p.dim && p.vdim <= p.dim && p.vdim % 8 == 0 &&
                p.dim % 8 == 0 && p.dim > 128 && p.dim <= 512 && !p.bias && p.softcap <= 0.f &&
                ((uintptr_t)p.kc & 15) == 0) {
       attn_latent_decode_kernel<1, AL_KC><<<grid, 64, 0, s>>>(p);
@@ -736,12 +861,13 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
       AB_BY_VREG(attn_bias_decode_kernel, grid, 64);
     }
     JLA_CHECK_LAUNCH();
-    attn_bias_merge_kernel<<<dim3(p.H, p.B, (p.vdim + 63) / 64), 64, 0, s>>>(p);
+    if (p.maps == 2) attn_diff_merge_kernel<<<dim3(p.H, p.B), (p.vdim + 63) / 64 * 64, 0, s>>>(p);
+    else attn_bias_merge_kernel<<<dim3(p.H, p.B, (p.vdim + 63) / 64), 64, 0, s>>>(p);
     JLA_CHECK_LAUNCH();
     return 0;
   }
   // (the flash kernel stores four columns at a time)
-  if (p.vt_ws && (p.S + 127) / 128 * (long long)p.H * p.B <= 0x7fffffffLL && p.ldv == p.vdim && p.ldo % 4 == 0 && ((uintptr_t)p.out & (p.out_bf16 ? 7 : 15)) == 0 &&
+  if (p.vt_ws && (p.S + 63) / 64 * (long long)p.H * p.B <= 0x7fffffffLL && p.ldv == p.vdim && p.ldk % 8 == 0 && p.ldo % 4 == 0 && ((uintptr_t)p.out & (p.out_bf16 ? 7 : 15)) == 0 &&
       hy_attn_prefill_ws_bytes(p.B, p.S, p.G, p.dim, p.vdim, p.T, p.cbf16) > 0) {
     const int Tp = (p.T + 31) / 32 * 32;
     bf16_t* vt = reinterpret_cast<bf16_t*>(p.vt_ws);
@@ -760,7 +886,8 @@ int hy_attn_bias(const AttnBias& p, hipStream_t s) {
     return -9;
   }
   dim3 grid((p.S + 3) / 4, p.H, p.B);
-  AB_BY_VREG(attn_bias_prefill_kernel, grid, 256);
+  if (p.maps == 2) AB_BY_VREG(attn_diff_prefill_kernel, grid, 256);
+  else AB_BY_VREG(attn_bias_prefill_kernel, grid, 256);
   JLA_CHECK_LAUNCH();
   return 0;
 }

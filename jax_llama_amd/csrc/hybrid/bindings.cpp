@@ -158,7 +158,7 @@ void route_topk(Tensor z, int64_t E, int64_t top, Tensor row_expert, Tensor row_
 
 void route_grouped(Tensor z, OptT correction, int64_t E, int64_t top, int64_t groups, int64_t keep, Tensor row_expert,
                    Tensor row_tok, Tensor row_w, OptT sort_tok, OptT sort_dst, OptT sort_w, OptT offs, bool sigmoid,
-                   int64_t group_top, bool normalise, double w_scale) {
+                   int64_t group_top, bool normalise, double w_scale, OptT z_bias) {
   check(z.dim() == 2 && z.size(1) >= E && top >= 1 && top <= E, "route_grouped: z is [M, >= E], 1 <= top <= E");
   int ldz = 0;
   const float* zp = rows2d(z, "z", z.size(1), &ldz);
@@ -166,12 +166,14 @@ void route_grouped(Tensor z, OptT correction, int64_t E, int64_t top, int64_t gr
   const int64_t R = (int64_t)M * top;
   check(row_w.numel() >= R, "route_grouped: weight outputs hold R numbers");
   check(!correction.has_value() || correction->numel() == E, "route_grouped: correction is [E]");
+  check(!z_bias.has_value() || z_bias->numel() == E, "route_grouped: z_bias is [E]");
   const bool sorted = sort_tok.has_value();
   check(sorted == sort_dst.has_value() && sorted == sort_w.has_value() && sorted == offs.has_value(),
         "route_grouped: the sorted outputs come together");
   check(!sorted || sort_w->numel() >= R, "route_grouped: weight outputs hold R numbers");
   rc(jla::hy_route_grouped(zp, ldz, correction.has_value() ? f32(*correction, "correction") : nullptr, M, top, E,
-                           jla::RouteRule{(int)groups, (int)keep, (int)group_top, sigmoid, normalise, (float)w_scale},
+                           jla::RouteRule{(int)groups, (int)keep, (int)group_top, sigmoid, normalise, (float)w_scale,
+                                          z_bias.has_value() ? f32(*z_bias, "z_bias") : nullptr},
                            i32w(row_expert, "row_expert", R), i32w(row_tok, "row_tok", R), f32w(row_w, "row_w"),
                            sorted ? i32w(*sort_tok, "sort_tok", R) : nullptr,
                            sorted ? i32w(*sort_dst, "sort_dst", R) : nullptr, sorted ? f32w(*sort_w, "sort_w") : nullptr,
@@ -273,11 +275,12 @@ void gelu_gate_rows(Tensor gp, Tensor ids, Tensor table, int64_t col0, Tensor g)
 void* slice2d_any(const Tensor& t, const char* name, int64_t rows, int64_t cols, int* ld, int* bf);
 
 void glu_rows(Tensor gu, Tensor out, int64_t act, double limit, double alpha) {
-  check(gu.dim() == 2 && out.dim() == 2 && gu.size(1) == 2 * out.size(1) && jla::hy_act_gated(act),
-        "glu_rows: gu is [M, 2F], out [M, F], a gated activation");
-  int ldo = 0, bf = 0;
+  check(gu.dim() == 2 && out.dim() == 2 && gu.size(1) >= 2 * out.size(1) && jla::hy_act_gated(act),
+        "glu_rows: gu is [M, >= 2F], out [M, F], a gated activation");
+  int ldg = 0, ldo = 0, bf = 0;
+  const float* gp = rows2d(gu, "gu", gu.size(1), &ldg);
   void* op = slice2d_any(out, "out", gu.size(0), out.size(1), &ldo, &bf);
-  rc(jla::hy_glu_rows(f32(gu, "gu"), gu.size(0), out.size(1), act, limit, alpha, op, bf, ldo, stream()), "glu_rows");
+  rc(jla::hy_glu_rows(gp, ldg, gu.size(0), out.size(1), act, limit, alpha, op, bf, ldo, stream()), "glu_rows");
 }
 
 // fp32 or bf16 dense [M, D] output
@@ -333,6 +336,42 @@ void depth_update(Tensor hist, int64_t i, bool store, Tensor x, Tensor x_out, do
     p.h = rows_out(*h, "h", md, &p.h_bf16);
   }
   rc(jla::hy_depth_update(p, stream()), "depth_update");
+}
+
+void sandwich_update(Tensor x, OptT y, int64_t nsum, OptT row_w, OptT bias, OptT extra, OptT post, double eps, OptT pre,
+                     OptT h) {
+  jla::SandwichUpdate p{};
+  check(x.dim() == 2, "sandwich_update: x is [M, D]");
+  p.M = x.size(0); p.D = x.size(1);
+  const int64_t md = (int64_t)p.M * p.D;
+  p.x = f32w(x, "x");
+  p.eps = eps;
+  p.nsum = nsum;
+  if (y.has_value()) {
+    check(nsum >= 1 && y->numel() == md * nsum, "sandwich_update: y is [M * nsum, D]");
+    check(post.has_value() && post->numel() == p.D, "sandwich_update: post is [D]");
+    p.y = f32(*y, "y");
+    p.post = f32(*post, "post");
+    if (row_w.has_value()) {
+      check(row_w->numel() >= (int64_t)p.M * nsum, "sandwich_update: row_w is [M * nsum]");
+      p.row_w = f32(*row_w, "row_w");
+    }
+    if (bias.has_value()) {
+      check(bias->numel() == p.D, "sandwich_update: bias is [D]");
+      p.bias = f32(*bias, "bias");
+    }
+    if (extra.has_value()) {
+      check(extra->numel() == md, "sandwich_update: extra is [M, D]");
+      p.extra = f32(*extra, "extra");
+    }
+  }
+  check(pre.has_value() == h.has_value(), "sandwich_update: pre and h together");
+  if (h.has_value()) {
+    check(pre->numel() == p.D, "sandwich_update: pre is [D]");
+    p.pre = f32(*pre, "pre");
+    p.h = rows_out(*h, "h", md, &p.h_bf16);
+  }
+  rc(jla::hy_sandwich_update(p, stream()), "sandwich_update");
 }
 
 void attn_prep(Tensor proj, Tensor positions, Tensor slot, int64_t B, int64_t S, int64_t H, int64_t G, int64_t dim,
@@ -426,14 +465,20 @@ int64_t attn_prefill_ws_bytes(int64_t B, int64_t S, int64_t G, int64_t dim, int6
 
 void attn_bias(Tensor q, Tensor kc, Tensor vc, Tensor slot, double scale, double softcap, OptT bias, Tensor out,
                int64_t t_cap, OptT ws, int64_t splits, OptT vt_ws, OptT sink, int64_t chunk, OptT head_scale, int64_t window,
-               int64_t keep_first, OptT gate, c10::optional<int64_t> vdim, bool gate_cols) {
+               int64_t keep_first, OptT gate, c10::optional<int64_t> vdim, bool gate_cols, int64_t maps, double diff_lambda,
+               double diff_eps, double diff_gain) {
   jla::AttnBias p{};
-  check(q.dim() == 4, "attn_bias: q is [B, S, H, dim]");
-  p.B = q.size(0); p.S = q.size(1); p.H = q.size(2); p.dim = q.size(3);
+  check(maps == 1 || maps == 2, "attn_bias: one or two maps per head");
+  check(q.dim() == 4 && q.size(2) % maps == 0, "attn_bias: q is [B, S, H * maps, dim]");
+  p.B = q.size(0); p.S = q.size(1); p.H = q.size(2) / maps; p.dim = q.size(3);
+  const int64_t qheads = q.size(2);
+  p.maps = maps;
+  p.ldk = maps * p.dim;
+  p.diff_lambda = diff_lambda; p.diff_eps = diff_eps; p.diff_gain = diff_gain;
   p.q = f32(q, "q");
   p.cbf16 = wtype(kc, "k cache");
   check(wtype(vc, "v cache") == p.cbf16, "attn_bias: cache dtypes differ");
-  check(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == p.B && vc.size(0) == p.B && kc.size(3) == p.dim &&
+  check(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == p.B && vc.size(0) == p.B && kc.size(3) == p.ldk &&
             kc.size(1) == vc.size(1) && kc.size(2) == vc.size(2),
         "attn_bias: cache shapes");
   p.G = kc.size(1); p.T = kc.size(2);
@@ -456,25 +501,25 @@ void attn_bias(Tensor q, Tensor kc, Tensor vc, Tensor slot, double scale, double
   p.scale = scale;
   p.softcap = softcap;
   if (bias.has_value()) {
-    check(bias->dim() == 2 && bias->size(1) == p.H, "attn_bias: bias is [distances, H]");
+    check(bias->dim() == 2 && bias->size(1) == qheads, "attn_bias: bias is [distances, query heads]");
     p.bias = f32(*bias, "bias");
     p.nbias = bias->size(0);
   }
   if (sink.has_value()) {
-    check(sink->numel() == p.H, "attn_bias: sink is [H]");
+    check(sink->numel() == qheads, "attn_bias: one sink per query head");
     p.sink = f32(*sink, "sink");
   }
   check(chunk >= 0 && chunk <= INT32_MAX, "attn_bias: chunk");
   p.chunk = chunk;
   if (head_scale.has_value()) {
-    check(head_scale->numel() == p.H, "attn_bias: head_scale is [H]");
+    check(head_scale->numel() == qheads, "attn_bias: one factor per query head");
     p.head_scale = f32(*head_scale, "head_scale");
   }
   p.out = slice2d_any(out, "out", (int64_t)p.B * p.S, (int64_t)p.H * p.vdim, &p.ldo, &p.out_bf16);
   p.t_cap = std::min<int64_t>(t_cap, p.T);
   p.splits = splits;
   if (p.S == 1) {
-    check(ws.has_value() && splits >= 1 && ws->numel() >= (int64_t)p.B * p.H * splits * (p.vdim + 2),
+    check(ws.has_value() && splits >= 1 && ws->numel() >= (int64_t)p.B * qheads * splits * (p.vdim + 2),
           "attn_bias: decode workspace");
     p.ws = f32w(*ws, "ws");
   }
@@ -645,10 +690,18 @@ void rope_prep(Tensor proj, OptT bias, Tensor positions, Tensor slot, int64_t B,
 }
 
 void qkv_prep(Tensor proj, OptT bias, OptT q_w, OptT k_w, double eps, Tensor positions, Tensor slot, int64_t B, int64_t S,
-              int64_t H, int64_t G, int64_t dim, int64_t vdim, Tensor kc, Tensor vc, Tensor q, OptT freq, bool halves,
-              OptT v_prev, OptT lambda, OptT v_out) {
+              int64_t H, int64_t G, int64_t dim, int64_t vdim, OptT kc, OptT vc, Tensor q, OptT freq, bool halves,
+              OptT v_prev, OptT lambda, OptT v_out, int64_t maps, bool v_is_k, double rot_gain) {
   jla::QkvPrep p{};
-  const int64_t cols = (H + G) * dim + G * vdim;
+  check(maps == 1 || maps == 2, "qkv_prep: one or two maps per head");
+  check(kc.has_value() == vc.has_value(), "qkv_prep: k and v caches together");
+  p.q_only = !kc.has_value();
+  p.maps = maps;
+  p.rot_gain = rot_gain;
+  check(!v_is_k || (vdim == maps * dim && !p.q_only), "qkv_prep: values that are the keys have their width");
+  const int64_t nq = H * maps * dim, nk = p.q_only ? 0 : G * maps * dim;
+  const int64_t cols = nq + nk + (p.q_only || v_is_k ? 0 : G * vdim);
+  p.v_col = v_is_k ? nq : nq + nk;
   check(proj.dim() == 2 && proj.size(0) == B * S && proj.size(1) >= cols, "qkv_prep: proj is [B * S, >= q | k | v columns]");
   p.proj = rows2d(proj, "proj", proj.size(1), &p.ld);
   if (bias.has_value()) {
@@ -656,26 +709,29 @@ void qkv_prep(Tensor proj, OptT bias, OptT q_w, OptT k_w, double eps, Tensor pos
     p.bias = f32(*bias, "bias");
   }
   if (q_w.has_value()) {
-    check(q_w->numel() == H * dim, "qkv_prep: q_w is [H * dim]");
+    check(q_w->numel() == nq, "qkv_prep: q_w has one gain per query column");
     p.q_w = f32(*q_w, "q_w");
   }
   if (k_w.has_value()) {
-    check(k_w->numel() == G * dim, "qkv_prep: k_w is [G * dim]");
+    check(k_w->numel() == nk, "qkv_prep: k_w has one gain per key column");
     p.k_w = f32(*k_w, "k_w");
   }
   p.eps = eps;
   p.positions = i32(positions, "positions", B * S);
   p.slot = i32(slot, "slot", 1);
   p.B = B; p.S = S; p.H = H; p.G = G; p.dim = dim; p.vdim = vdim;
-  p.cbf16 = wtype(kc, "k cache");
-  check(wtype(vc, "v cache") == p.cbf16, "qkv_prep: cache dtypes differ");
-  check(kc.dim() == 4 && kc.size(0) == B && kc.size(1) == G && kc.size(3) == dim, "qkv_prep: k cache shape");
-  p.T = kc.size(2);
-  check(vc.dim() == 4 && vc.size(0) == B && vc.size(1) == G && vc.size(2) == p.T && vc.size(3) == vdim,
-        "qkv_prep: v cache shape");
-  p.kc = kc.data_ptr();
-  p.vc = vc.data_ptr();
-  check(q.numel() == B * S * H * dim, "qkv_prep: q shape");
+  p.T = 1;
+  if (!p.q_only) {
+    p.cbf16 = wtype(*kc, "k cache");
+    check(wtype(*vc, "v cache") == p.cbf16, "qkv_prep: cache dtypes differ");
+    check(kc->dim() == 4 && kc->size(0) == B && kc->size(1) == G && kc->size(3) == maps * dim, "qkv_prep: k cache shape");
+    p.T = kc->size(2);
+    check(vc->dim() == 4 && vc->size(0) == B && vc->size(1) == G && vc->size(2) == p.T && vc->size(3) == vdim,
+          "qkv_prep: v cache shape");
+    p.kc = kc->data_ptr();
+    p.vc = vc->data_ptr();
+  }
+  check(q.numel() == B * S * nq, "qkv_prep: q shape");
   p.q = f32w(q, "q");
   if (freq.has_value() && freq->numel() > 0) {
     p.half = freq->numel();
@@ -782,7 +838,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route_grouped", &route_grouped, py::arg("z"), py::arg("correction"), py::arg("E"), py::arg("top"),
         py::arg("groups"), py::arg("keep"), py::arg("row_expert"), py::arg("row_tok"), py::arg("row_w"),
         py::arg("sort_tok"), py::arg("sort_dst"), py::arg("sort_w"), py::arg("offs"), py::arg("sigmoid") = false,
-        py::arg("group_top") = 1, py::arg("normalise") = false, py::arg("w_scale") = 1.0);
+        py::arg("group_top") = 1, py::arg("normalise") = false, py::arg("w_scale") = 1.0,
+        py::arg("z_bias") = py::none());
   m.def("hc_update", &hc_update);
   m.def("linear_rows", &linear_rows, py::arg("a"), py::arg("a_idx"), py::arg("w"), py::arg("out"), py::arg("dst_idx"),
         py::arg("offs"), py::arg("row_expert"), py::arg("R"), py::arg("act"), py::arg("act_limit"), py::arg("act_alpha"),
@@ -812,7 +869,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("softcap"), py::arg("bias"), py::arg("out"), py::arg("t_cap"), py::arg("ws"), py::arg("splits"),
         py::arg("vt_ws"), py::arg("sink"), py::arg("chunk") = 0, py::arg("head_scale") = py::none(),
         py::arg("window") = 0, py::arg("keep_first") = 0, py::arg("gate") = py::none(), py::arg("vdim") = py::none(),
-        py::arg("gate_cols") = false);
+        py::arg("gate_cols") = false, py::arg("maps") = 1, py::arg("diff_lambda") = 0.0, py::arg("diff_eps") = 0.0,
+        py::arg("diff_gain") = 1.0);
   m.def("attn_prefill_ws_bytes", &attn_prefill_ws_bytes);
   m.def("delta_prep", &delta_prep);
   m.def("conv_state_update", &conv_state_update);
@@ -825,7 +883,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("qkv_prep", &qkv_prep, py::arg("proj"), py::arg("bias"), py::arg("q_w"), py::arg("k_w"), py::arg("eps"),
         py::arg("positions"), py::arg("slot"), py::arg("B"), py::arg("S"), py::arg("H"), py::arg("G"), py::arg("dim"),
         py::arg("vdim"), py::arg("kc"), py::arg("vc"), py::arg("q"), py::arg("freq"), py::arg("halves") = false,
-        py::arg("v_prev") = py::none(), py::arg("lambda_") = py::none(), py::arg("v_out") = py::none());
+        py::arg("v_prev") = py::none(), py::arg("lambda_") = py::none(), py::arg("v_out") = py::none(),
+        py::arg("maps") = 1, py::arg("v_is_k") = false, py::arg("rot_gain") = 1.0);
+  m.def("sandwich_update", &sandwich_update);
   m.def("glu_rows", &glu_rows);
   m.def("squash_rows", &squash_rows);
   m.def("depth_update", &depth_update);

@@ -83,12 +83,13 @@ int hy_route_topk(const float* z, int ldz, int M, int top, int E, int32_t* row_e
 // (correction optional); the E experts form `groups` equal groups of neighbours, a group's score is the sum of its
 // `group_top` (1 or 2) largest choice scores, and only experts of the `keep` best groups can be chosen; the `top` largest
 // are taken (ties to the lower index everywhere), weight = w_scale * the chosen expert's score, with normalise also
-// divided by (the chosen scores' sum + 1e-20). Same outputs as hy_route_topk. E <= 1024, E % groups == 0, groups <= 64,
-// top <= keep * (E / groups).
+// divided by (the chosen scores' sum + 1e-20). z_bias (optional) joins the logits (choice and weights). Same outputs as
+// hy_route_topk. E <= 1024, E % groups == 0, groups <= 64, top <= keep * (E / groups).
 struct RouteRule {
   int groups, keep, group_top;
   int sigmoid, normalise;
   float w_scale;
+  const float* z_bias;  // [E] or nullptr
 };
 int hy_route_grouped(const float* z, int ldz, const float* correction, int M, int top, int E, RouteRule rule,
                      int32_t* row_expert, int32_t* row_tok, float* row_w, int32_t* sort_tok, int32_t* sort_dst,
@@ -128,9 +129,9 @@ int hy_norm_residual(const float* y, int nsum, float ysc, const float* w, int w_
 typedef uint16_t bf16_t;
 int hy_cast_bf16(const float* x, bf16_t* y, long long n, int act, hipStream_t s);
 
-// out[m * ldo + c] = act(gu[m, c], gu[m, F + c]) for c < F: the gated epilogue of a product [M, 2F] that ran on the packed
-// GEMM; out fp32 or bf16, a column slice
-int hy_glu_rows(const float* gu, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
+// out[m * ldo + c] = act(gu[m * ldg + c], gu[m * ldg + F + c]) for c < F: the gated epilogue of a product [M, >= 2F] that ran
+// on the packed GEMM; out fp32 or bf16, a column slice
+int hy_glu_rows(const float* gu, int ldg, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
                 hipStream_t s);
 
 // h = tanh(alpha * x) * w + b, element by element (alpha one number, w and b [D]); h fp32 or bf16
@@ -159,6 +160,27 @@ struct DepthUpdate {
   int h_bf16;
 };
 int hy_depth_update(const DepthUpdate& p, hipStream_t s);
+
+// The residual step between two sublayers of a stack with norms on both sides of each: with
+//   v = y[m] (nsum == 1 without row_w), or sum_{c < nsum} w_c y[m * nsum + c] (w_c = row_w[m * nsum + c], absent: 1),
+//       [+ bias] [+ extra[m]],
+//   x[m] += v / sqrt(mean(v^2) + eps) * post;   h[m] = x[m] / sqrt(mean(x[m]^2) + eps) * pre   (with h)
+// y == nullptr: only h.
+struct SandwichUpdate {
+  float* x;  // [M, D], read and written
+  int M, D;
+  const float* y;
+  int nsum;
+  const float* row_w;  // optional [M * nsum]
+  const float* bias;   // optional [D]
+  const float* extra;  // optional [M, D]
+  const float* post;   // [D]
+  float eps;
+  const float* pre;    // [D], with h
+  void* h;             // optional [M, D] fp32 or bf16
+  int h_bf16;
+};
+int hy_sandwich_update(const SandwichUpdate& p, hipStream_t s);
 
 // x <- cap * tanh(x / cap) in place (cap = 1: tanh), n elements
 int hy_softcap(float* x, long long n, float cap, hipStream_t s);
@@ -215,9 +237,9 @@ struct LatentPrep {
 int hy_latent_prep(const LatentPrep& p, hipStream_t s);
 
 struct AttnBias {
-  const float* q;  // [B, S, H, dim]
-  const void* kc;
-  const void* vc;
+  const float* q;  // [B, S, H * maps, dim]
+  const void* kc;  // [B, G, T, ldk]: key rows, the maps of a head side by side
+  const void* vc;  // [B, G, T, ldv]
   int cbf16;
   const int32_t* slot;
   int B, S, H, G, dim, vdim, T;
@@ -240,6 +262,11 @@ struct AttnBias {
   int ldg;            // (gate_cols) its column c by sigmoid(gate[m * ldg + h * vdim + c])
   int gate_cols;
   int ldv;         // elements between value rows (>= vdim; the values are the first vdim numbers of each row)
+  int ldk;         // elements between key rows (>= maps * dim)
+  int maps;        // 1, or 2 (differential heads): query head 2 h + b attends with map b of head h's key rows, the output is
+                   // d / sqrt(mean(d^2) + diff_eps) * diff_gain with d = a_0 - diff_lambda * a_1 over the head's vdim
+                   // numbers; sink, head_scale and bias columns are per query head, gates per output head; the decode
+  float diff_lambda, diff_eps, diff_gain;  // partials take B * H * maps * splits * (vdim + 2) floats
 };
 int hy_attn_bias(const AttnBias& p, hipStream_t s);
 long long hy_attn_prefill_ws_bytes(int B, int S, int G, int dim, int vdim, int T, int cbf16);
@@ -323,22 +350,27 @@ int hy_rope_prep(const RopePrep& p, hipStream_t s);
 struct QkvPrep {
   const float* proj;  // [M, ld]: q heads, k heads, v heads (more columns may follow)
   int ld;
-  const float* bias;  // optional [H dim + G dim + G vdim]
-  const float* q_w;   // optional [H dim] (absent: no norm)
-  const float* k_w;   // optional [G dim]
+  const float* bias;  // optional, one per column in use
+  const float* q_w;   // optional [H maps dim] (absent: no norm)
+  const float* k_w;   // optional [G maps dim]
   float eps;
   const int32_t* positions;  // [M]
   const int32_t* slot;
   int B, S, H, G, dim, vdim, T;
-  void* kc;  // [B, G, T, dim]
+  void* kc;  // [B, G, T, maps * dim]
   void* vc;  // [B, G, T, vdim]
   int cbf16;
-  float* q;  // [M, H, dim]
+  float* q;  // [M, H * maps, dim]
   const double* freq;  // [half]
   int half, halves;
   const float* v_prev;  // optional [M, G vdim], with lambda
   const float* lambda;  // [1]
   float* v_out;         // optional [M, G vdim]: the values as cached, in fp32
+  int maps;             // dim-sized parts of a head's q and k, each rotated by itself (1 or 2); a key row holds them side by
+                        // side, q has H * maps heads
+  int v_col;            // column of the first value (values that are the keys as projected: H maps dim)
+  float rot_gain;       // factor on every cosine and sine
+  int q_only;           // 1: proj holds q alone, nothing is cached (the layer reads another layer's keys and values)
 };
 int hy_qkv_prep(const QkvPrep& p, hipStream_t s);
 

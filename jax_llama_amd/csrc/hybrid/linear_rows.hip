@@ -580,7 +580,7 @@ __global__ void __launch_bounds__(256) route_grouped_select_kernel(const float* 
 #pragma unroll
   for (int u = 0; u < RK_PER_LANE; ++u) {
     const int e = lane + 64 * u;
-    const float f = e < E ? zr[e] : -INFINITY;
+    const float f = e < E ? zr[e] + (rule.z_bias ? rule.z_bias[e] : 0.f) : -INFINITY;
     sc[u] = f == f ? f : -INFINITY;  // (a NaN logit counts as minus infinity)
     zmax = fmaxf(zmax, sc[u]);
   }
@@ -681,7 +681,7 @@ __global__ void __launch_bounds__(256) route_grouped_select64_kernel(const float
   const int groups = rule.groups, keep = rule.keep;
   if (m >= M) return;
   const bool valid = lane < E;
-  float zv = valid ? z[(size_t)m * ldz + lane] : -INFINITY;
+  float zv = valid ? z[(size_t)m * ldz + lane] + (rule.z_bias ? rule.z_bias[lane] : 0.f) : -INFINITY;
   const float cr = valid && correction ? correction[lane] : 0.f;
   zv = zv == zv ? zv : -INFINITY;
   float sc;

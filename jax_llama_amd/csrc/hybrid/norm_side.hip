@@ -3,7 +3,8 @@
 // (gelu_tanh(gate projection) * a slice of a second embedding table), the latent-attention prep (normed latent, normed
 // query latent, rotated shared key part, cache write), the hyper-connection update of several residual streams, and the
 // residual step of a depth-averaging stack (residual add, weighted sum of every earlier layer's result, the next layer's
-// statistics-free norm: everything is element by element, so one pass serves all three).
+// statistics-free norm: everything is element by element, so one pass serves all three), and the residual step of a stack
+// with norms on both sides of every sublayer (output norm, residual add and the next sublayer's input norm in one pass).
 // fp32 statistics and residual.
 #include "hy_util.h"
 #include "hybrid.h"
@@ -535,7 +536,7 @@ int hy_squash_rows(const float* x, int M, int D, const float* alpha, const float
 
 // V columns of one token per thread: the gated activation of a product whose gate and up columns lie side by side
 template <int V>
-__global__ void __launch_bounds__(256) glu_rows_kernel(const float* __restrict__ gu, int F, int act, float limit,
+__global__ void __launch_bounds__(256) glu_rows_kernel(const float* __restrict__ gu, int ldg, int F, int act, float limit,
                                                        float alpha, void* out, int out_bf16, int ldo, long long n) {
   const long long t = (long long)blockIdx.x * 256 + threadIdx.x;
   if (t >= n) return;
@@ -543,8 +544,8 @@ __global__ void __launch_bounds__(256) glu_rows_kernel(const float* __restrict__
   const long long m = t / fv;
   const int c = (int)(t - m * fv) * V;
   float g[V], u[V];
-  dv_load<V>(gu + (size_t)m * 2 * F + c, g);
-  dv_load<V>(gu + (size_t)m * 2 * F + F + c, u);
+  dv_load<V>(gu + (size_t)m * ldg + c, g);
+  dv_load<V>(gu + (size_t)m * ldg + F + c, u);
 #pragma unroll
   for (int k = 0; k < V; ++k) {
     if (act == HY_ACT_SWIGLU) {
@@ -559,17 +560,141 @@ __global__ void __launch_bounds__(256) glu_rows_kernel(const float* __restrict__
   dv_store_h<V>(out, out_bf16, (size_t)m * ldo + c, g);
 }
 
-int hy_glu_rows(const float* gu, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
+int hy_glu_rows(const float* gu, int ldg, int M, int F, int act, float limit, float alpha, void* out, int out_bf16, int ldo,
                 hipStream_t s) {
-  if (M < 0 || F < 1 || ldo < F || !hy_act_gated(act)) return -1;
+  if (M < 0 || F < 1 || ldo < F || ldg < 2 * F || !hy_act_gated(act)) return -1;
   if (M == 0) return 0;
   const uintptr_t mask = out_bf16 ? 7 : 15;
-  const int v = F % 4 == 0 && ldo % 4 == 0 && ((uintptr_t)out & mask) == 0 ? 4 : 1;
+  const int v = F % 4 == 0 && ldg % 4 == 0 && ldo % 4 == 0 && (((uintptr_t)out & mask) | ((uintptr_t)gu & 15)) == 0 ? 4 : 1;
   const long long n = (long long)M * (F / v);
   if ((n + 255) / 256 > 0x7fffffffLL) return -2;
   const unsigned grid = (unsigned)((n + 255) / 256);
-  if (v == 4) glu_rows_kernel<4><<<grid, 256, 0, s>>>(gu, F, act, limit, alpha, out, out_bf16, ldo, n);
-  else glu_rows_kernel<1><<<grid, 256, 0, s>>>(gu, F, act, limit, alpha, out, out_bf16, ldo, n);
+  if (v == 4) glu_rows_kernel<4><<<grid, 256, 0, s>>>(gu, ldg, F, act, limit, alpha, out, out_bf16, ldo, n);
+  else glu_rows_kernel<1><<<grid, 256, 0, s>>>(gu, ldg, F, act, limit, alpha, out, out_bf16, ldo, n);
+  JLA_CHECK_LAUNCH();
+  return 0;
+}
+
+// ---- norms on both sides of every sublayer -----------------------------------------------------------------------------
+// One workgroup per token. NV > 0: a thread owns NV groups of four columns 1024 apart (a template parameter: the sublayer's
+// rows, the residual, the gains, all branch-free and in flight together; surplus threads re-read the last group and count
+// nothing); the row stays in registers between the two statistics. NV = 0: any width, walks of single columns.
+template <int NV>
+__global__ void __launch_bounds__(256) sandwich_update_kernel(SandwichUpdate p) {
+  __shared__ float red[16];
+  const int m = blockIdx.x, tid = threadIdx.x, D = p.D;
+  const size_t row = (size_t)m * D;
+  const float* yr = p.y ? p.y + row * p.nsum : nullptr;
+  const float* rw = p.row_w ? p.row_w + (size_t)m * p.nsum : nullptr;
+  if constexpr (NV > 0) {
+    float x[NV][4], v[NV][4], po[NV][4], pr[NV][4];
+    int dd[NV];
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      dd[u] = min(4 * tid + 1024 * u, D - 4);
+      dv_load<4>(p.x + row + dd[u], x[u]);
+      if (p.h) dv_load<4>(p.pre + dd[u], pr[u]);
+    }
+    if (yr) {
+#pragma unroll
+      for (int u = 0; u < NV; ++u) {
+        dv_load<4>(p.post + dd[u], po[u]);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[u][k] = 0.f;
+        if (p.bias) dv_load<4>(p.bias + dd[u], v[u]);
+        if (p.extra) {
+          float e[4];
+          dv_load<4>(p.extra + row + dd[u], e);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) v[u][k] += e[k];
+        }
+      }
+#pragma unroll 2
+      for (int c = 0; c < p.nsum; ++c) {
+        const float w = rw ? rw[c] : 1.f;
+#pragma unroll
+        for (int u = 0; u < NV; ++u) {
+          float f[4];
+          dv_load<4>(yr + (size_t)c * D + dd[u], f);
+#pragma unroll
+          for (int k = 0; k < 4; ++k) v[u][k] = fmaf(w, f[k], v[u][k]);
+        }
+      }
+      float ss = 0.f;
+#pragma unroll
+      for (int u = 0; u < NV; ++u)
+        if (4 * tid + 1024 * u < D)
+#pragma unroll
+          for (int k = 0; k < 4; ++k) ss = fmaf(v[u][k], v[u][k], ss);
+      const float sc = 1.f / sqrtf(block_sum(ss, red) / (float)D + p.eps);
+#pragma unroll
+      for (int u = 0; u < NV; ++u) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) x[u][k] += v[u][k] * sc * po[u][k];
+        if (4 * tid + 1024 * u < D) dv_store<4>(p.x + row + dd[u], x[u]);
+      }
+    }
+    if (!p.h) return;
+    float ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u)
+      if (4 * tid + 1024 * u < D)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) ss = fmaf(x[u][k], x[u][k], ss);
+    const float sc = 1.f / sqrtf(block_sum(ss, red) / (float)D + p.eps);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) x[u][k] = x[u][k] * sc * pr[u][k];
+      if (4 * tid + 1024 * u < D) dv_store_h<4>(p.h, p.h_bf16, row + dd[u], x[u]);
+    }
+    return;
+  }
+  auto value = [&](int d) {
+    float v = (p.bias ? p.bias[d] : 0.f) + (p.extra ? p.extra[row + d] : 0.f);
+    for (int c = 0; c < p.nsum; ++c) v = fmaf(rw ? rw[c] : 1.f, yr[(size_t)c * D + d], v);
+    return v;
+  };
+  float sc = 0.f, sx = 0.f;
+  if (yr) {
+    float ss = 0.f;
+    for (int d = tid; d < D; d += 256) {
+      const float v = value(d);
+      ss = fmaf(v, v, ss);
+    }
+    sc = 1.f / sqrtf(block_sum(ss, red) / (float)D + p.eps);
+  }
+  for (int d = tid; d < D; d += 256) {
+    float x = p.x[row + d];
+    if (yr) {
+      x += value(d) * sc * p.post[d];
+      p.x[row + d] = x;
+    }
+    sx = fmaf(x, x, sx);
+  }
+  if (!p.h) return;
+  const float sn = 1.f / sqrtf(block_sum(sx, red) / (float)D + p.eps);
+  for (int d = tid; d < D; d += 256) {  // (a thread reads back the columns it wrote)
+    const float h = p.x[row + d] * sn * p.pre[d];
+    dv_store_h<1>(p.h, p.h_bf16, row + d, &h);
+  }
+}
+
+int hy_sandwich_update(const SandwichUpdate& p, hipStream_t s) {
+  if (p.M < 0 || p.D < 1 || !p.x || (!p.y && !p.h)) return -1;
+  if (p.y && (!p.post || p.nsum < 1)) return -2;
+  if (p.h && !p.pre) return -3;
+  if (p.M == 0) return 0;
+  const uintptr_t at = (uintptr_t)p.x | (uintptr_t)p.y | (uintptr_t)p.bias | (uintptr_t)p.extra | (uintptr_t)p.post |
+                       (uintptr_t)p.pre | (uintptr_t)p.h;
+  const int nv = p.D % 4 || (at & 15) ? 0 : (p.D + 1023) / 1024;
+#define SU_LAUNCH(NV) sandwich_update_kernel<NV><<<p.M, 256, 0, s>>>(p)
+  if (nv == 0 || nv > 8) SU_LAUNCH(0);
+  else if (nv == 1) SU_LAUNCH(1);
+  else if (nv == 2) SU_LAUNCH(2);
+  else if (nv <= 4) SU_LAUNCH(4);
+  else SU_LAUNCH(8);
+#undef SU_LAUNCH
   JLA_CHECK_LAUNCH();
   return 0;
 }

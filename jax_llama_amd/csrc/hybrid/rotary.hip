@@ -12,7 +12,9 @@
 //                     interleaved layout: the rotated tail of a latent attention's queries, in place).
 //   hy_qkv_prep     : the step after a fused q | k | v projection whose RMS norms run over the whole q and the whole k
 //                     (before they are split into heads), with both pair layouts, and values blended with the same
-//                     token's values of another layer.
+//                     token's values of another layer. Heads may hold two maps (each rotated by itself), the values may
+//                     be the key columns as projected, cosine and sine may carry a factor, and a layer may bring
+//                     queries only.
 #include "hy_util.h"
 #include "hybrid.h"
 
@@ -96,7 +98,8 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
   const int tid = threadIdx.x;
   const int m = blockIdx.x, b = m / p.S, t = *p.slot + (m - b * p.S);
   const float* row = p.proj + (size_t)m * p.ld;
-  const int nq = p.H * p.dim, nk = p.G * p.dim;
+  const int qh = p.H * p.maps, kh = p.q_only ? 0 : p.G * p.maps;  // dim-sized parts of q and k
+  const int nq = qh * p.dim, nk = kh * p.dim, ldk = p.maps * p.dim;
   const int pos = p.half > 0 ? p.positions[m] : 0;
   // both sums of squares in one walk over q | k, eight loads of a thread in flight, and the angle table behind them
   float sq = 0.f, sk = 0.f;
@@ -116,7 +119,12 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
       }
     }
   }
-  for (int i = tid; i < p.half; i += 256) ro_sincos(pos, p.freq[i], 1.f, &sn[i], &cs[i]);
+  for (int i = tid; i < p.half; i += 256) {
+    float si, co;
+    ro_sincos(pos, p.freq[i], 1.f, &si, &co);
+    sn[i] = si * p.rot_gain;
+    cs[i] = co * p.rot_gain;
+  }
   sq = wave_sum(sq);
   sk = wave_sum(sk);
   if ((tid & 63) == 0) {
@@ -132,7 +140,7 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
   const float lam = p.v_prev ? *p.lambda : 0.f;
   // q / k: an item is a rotated pair or a number that passes, (dim - half) of them per head; values: one number each. A
   // thread's items are taken QP_UNR at a time, all of their loads before the first use.
-  const int per = p.dim - p.half, n_qk = (p.H + p.G) * per, n_v = p.G * p.vdim;
+  const int per = p.dim - p.half, n_qk = (qh + kh) * per, n_v = p.q_only ? 0 : p.G * p.vdim;
   const int step = gridDim.y * 256, first = blockIdx.y * 256 + tid;
   for (int i0 = first; i0 < n_qk; i0 += QP_UNR * step) {
     float u[QP_UNR], v[QP_UNR];
@@ -146,7 +154,7 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
       du[k] = i < p.half ? (p.halves ? i : 2 * i) : i + p.half;
       dv[k] = i < p.half ? (p.halves ? i + p.half : 2 * i + 1) : du[k];
       const int cu = head[k] * p.dim + du[k], cv = head[k] * p.dim + dv[k];
-      const bool is_q = head[k] < p.H;
+      const bool is_q = head[k] < qh;
       const float* gw = is_q ? p.q_w : (p.k_w ? p.k_w - nq : nullptr);
       const float rs = is_q ? rq : rk;
       u[k] = (row[cu] + (p.bias ? p.bias[cu] : 0.f)) * rs * (gw ? gw[cu] : 1.f);
@@ -161,12 +169,13 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
         a = u[k] * co - v[k] * si;
         c = v[k] * co + u[k] * si;
       }
-      if (head[k] < p.H) {
+      if (head[k] < qh) {
         float* qd = p.q + (size_t)m * nq + head[k] * p.dim;
         qd[du[k]] = a;
         if (pair[k] >= 0) qd[dv[k]] = c;
       } else if (store) {
-        CT* cd = reinterpret_cast<CT*>(p.kc) + (((size_t)b * p.G + (head[k] - p.H)) * p.T + t) * p.dim;
+        const int part = head[k] - qh, g = part / p.maps;
+        CT* cd = reinterpret_cast<CT*>(p.kc) + (((size_t)b * p.G + g) * p.T + t) * ldk + (part - g * p.maps) * p.dim;
         ro_st(cd + du[k], a);
         if (pair[k] >= 0) ro_st(cd + dv[k], c);
       }
@@ -176,7 +185,7 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
     float v[QP_UNR], vp[QP_UNR];
 #pragma unroll
     for (int k = 0; k < QP_UNR; ++k) {
-      const int d = min(i0 + k * step, n_v - 1), c = nq + nk + d;
+      const int d = min(i0 + k * step, n_v - 1), c = p.v_col + d;
       v[k] = row[c] + (p.bias ? p.bias[c] : 0.f);
       vp[k] = p.v_prev ? p.v_prev[(size_t)m * n_v + d] : 0.f;
     }
@@ -195,12 +204,15 @@ __global__ void __launch_bounds__(256) qkv_prep_kernel(QkvPrep p) {
 int hy_qkv_prep(const QkvPrep& p, hipStream_t s) {
   if (p.B < 0 || p.S < 1 || p.H < 1 || p.G < 1 || p.H % p.G || p.dim < 1 || p.vdim < 1 || p.T < 1) return -1;
   if (p.half < 0 || 2 * p.half > p.dim || p.half > QP_MAX_HALF || (p.half > 0 && !p.freq)) return -2;
-  if ((long long)(p.H + p.G) * p.dim + (long long)p.G * p.vdim > p.ld) return -3;
+  if (p.maps != 1 && p.maps != 2) return -6;
+  const int parts = (p.H + (p.q_only ? 0 : p.G)) * p.maps;
+  if ((long long)parts * p.dim > p.ld || (!p.q_only && (p.v_col < 0 || (long long)p.v_col + p.G * p.vdim > p.ld))) return -3;
+  if (!p.q_only && (!p.kc || !p.vc)) return -7;
   if (p.v_prev && !p.lambda) return -4;
   const long long M = (long long)p.B * p.S;
   if (M == 0) return 0;
   if (M > 0x7fffffffLL) return -5;
-  const dim3 grid((unsigned)M, M <= 8 ? (unsigned)min(8, ((p.H + p.G) * (p.dim - p.half) + 255) / 256) : 1u);
+  const dim3 grid((unsigned)M, M <= 8 ? (unsigned)min(8, (parts * (p.dim - p.half) + 255) / 256) : 1u);
   if (p.cbf16) qkv_prep_kernel<bf16_t><<<grid, 256, 0, s>>>(p);
   else qkv_prep_kernel<float><<<grid, 256, 0, s>>>(p);
   JLA_CHECK_LAUNCH();

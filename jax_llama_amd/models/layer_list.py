@@ -46,6 +46,7 @@ class LayerListLM:
         self.embed_norm: Optional[torch.Tensor] = None  # fp32 [D]: gain of an RMS norm on the embedding
         self.logit_softcap = 0.0                        # logits <- cap * tanh(logits / cap) when > 0
         self.depth_history = False  # the blocks average over all layers' results (mixers.DepthAverageBlock)
+        self.chained_norms = False  # a block leaves the next one's normed input behind (mixers.SandwichChainBlock)
         self.streams = 0  # > 0: the blocks work on that many residual streams [S, M, D] (hyper-connections)
         self.final_norm = None  # gain of the last RMS norm (fp32, one number or [D]), or an hy.SquashNorm
         self.head: Optional[torch.Tensor] = None
@@ -152,6 +153,16 @@ class LayerListLM:
                 blk(x, ctx)
                 if collect_hidden:
                     hidden.append(x.reshape(b, s, d).clone())
+        elif self.chained_norms:
+            x = hy.embed_rows(idf, self.embed, scale=self.embed_scale)
+            ctx.act_dtype = BF16 if hy.prompt_bf16(b * s, d, self.param_dtype) else F32
+            ctx.every_row = logits_mode == "all" or (s == 1 and logits_mode in ("last", "argmax"))
+            if self.blocks:
+                ctx.h = hy.sandwich_update_(x, None, None, self.eps, pre=self.blocks[0].pre1, h_dtype=ctx.act_dtype)
+            for blk in self.blocks:
+                blk(x, ctx)
+                if collect_hidden:
+                    hidden.append(x.reshape(b, s, d).clone())
         else:
             x = hy.embed_rows(idf, self.embed, scale=self.embed_scale)
             if self.embed_norm is not None:
@@ -173,6 +184,8 @@ class LayerListLM:
         cap = float(self.logit_softcap or 0.0)
         if isinstance(self.final_norm, hy.SquashNorm):
             xf = ctx.h if ctx.every_row and ctx.h is not None else hy.squash_rows(xl, self.final_norm)
+        elif self.chained_norms and ctx.every_row and ctx.h is not None:
+            xf = ctx.h
         else:
             xf = hy.rms_rows(xl, self.final_norm, self.eps)
         logits = hy.linear(xf, self.head,

@@ -42,6 +42,11 @@ the same mechanisms with other values.
   DepthAverageBlock : mixer and feed-forward side by side on one statistics-free norm; the layer's result joins a history
                     of all layers' results, and the next layer reads a weighted sum of them.
 
+  DifferentialAttention : two softmax maps per head over the same values, their weighted difference RMS-normed per head; may
+                    read another layer's keys and values.
+  SharedExpertMoE : gated experts chosen by a biased softmax router (weights over the chosen logits), a shared expert.
+  SandwichChainBlock : the sandwich-norm residual in one kernel per sublayer, which also leaves the next sublayer's input.
+
 The mixers of the last group split into ``features(proj, ctx, out)`` -- everything between the fused input projection
 ``w_in`` and the output matrix ``w_o`` -- so that their block can fuse other rows (a router) into the input product and run
 one output product over the features of all of its members.
@@ -236,6 +241,7 @@ class FFOut:
     nsum: int = 1
     extra: Optional[torch.Tensor] = None
     extra_gate: Optional[torch.Tensor] = None
+    row_w: Optional[torch.Tensor] = None  # [M * nsum]: weights of the summed rows (absent: 1)
 
 
 class DenseFF:
@@ -638,17 +644,20 @@ class WholeNormAttention:
     softmax denominator (zeros: a constant one beside the exponentials). ``lam``: the values are blended with the first
     value-mixing layer's of the same token before they are cached, ``v <- (1 - lam) v + lam v_first``; that first layer
     (``lam`` None, ``leads``) leaves its values in the step's context. ``gated``: every output column is multiplied by the
-    sigmoid of a projection column of its own. The output projection's bias is ``o_bias``."""
+    sigmoid of a projection column of its own. The output projection's bias is ``o_bias``. ``v_is_k``: no value projection,
+    the values are the keys as projected (with bias, before norm and rotation); ``rot_gain``: a factor on cosine and sine."""
 
     def __init__(self, layer_idx: int, spec, eps: float, w_in: torch.Tensor, bias: Optional[torch.Tensor],
                  q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], freq: Optional[torch.Tensor],
                  sink: Optional[torch.Tensor], leads: bool, lam: Optional[torch.Tensor], w_o: torch.Tensor,
-                 o_bias: Optional[torch.Tensor], gated: bool = True, interleaved: bool = True):
+                 o_bias: Optional[torch.Tensor], gated: bool = True, interleaved: bool = True, v_is_k: bool = False,
+                 rot_gain: float = 1.0):
         self.i = layer_idx
         self.spec = spec
         self.eps = eps
-        self.w_in = w_in    # [H dim + G dim + G vdim (+ H vdim), D]: q | k | v | gates
-        self.bias = bias    # fp32 [H dim + G dim + G vdim] or None
+        self.w_in = w_in    # [H dim + G dim (+ G vdim) (+ H vdim), D]: q | k | v | gates
+        self.bias = bias    # fp32, one per q / k / v column, or None
+        self.v_is_k, self.rot_gain = v_is_k, rot_gain
         self.q_norm, self.k_norm = q_norm, k_norm  # fp32 [H dim], [G dim]
         self.freq = freq    # float64 [rot_dims / 2] or None
         self.sink = sink    # fp32 [H] or None
@@ -662,10 +671,11 @@ class WholeNormAttention:
         kc, vc = ctx.cache.layer(self.i)
         q, v = hy.qkv_prep(proj, self.bias, self.q_norm, self.k_norm, self.eps, ctx.positions, ctx.slot0, ctx.b, ctx.s,
                            sp.heads, sp.kv_heads, sp.dim, sp.vdim, kc, vc, self.freq, self.interleaved,
-                           ctx.v_first if self.lam is not None else None, self.lam, self.leads)
+                           ctx.v_first if self.lam is not None else None, self.lam, self.leads, v_is_k=self.v_is_k,
+                           rot_gain=self.rot_gain)
         if self.leads:
             ctx.v_first = v
-        c = (sp.heads + sp.kv_heads) * sp.dim + sp.kv_heads * sp.vdim
+        c = (sp.heads + sp.kv_heads) * sp.dim + (0 if self.v_is_k else sp.kv_heads * sp.vdim)
         gate = proj[:, c:c + self.width] if self.gated else None
         return hy.attn_bias(q, kc, vc, ctx.slot0, sp.scale, sink=self.sink, window=sp.window, gate=gate, gate_cols=True,
                             out=out)
@@ -759,3 +769,101 @@ class DepthAverageBlock:
         ctx.h = hy.depth_update_(ctx.hist, self.i, ctx.hist[0] if self.i == 0 else x, x, self.mult, y, self.coef,
                                  self.mixer.o_bias, ye, self.moe.top if self.moe is not None else 1, row_w, not self.last,
                                  norm, ctx.act_dtype)
+
+
+class DifferentialAttention:
+    """Softmax attention with two maps per head. q and k hold ``2 dim`` numbers per head (map 1, map 2; a cached key row
+    likewise), each map rotated by itself on its first ``2 len(freq)`` numbers (pairs ``i``, ``i + len(freq)``) and attending
+    causally over the same values; a head's output is the first map's minus ``lam`` times the second's, divided by its root
+    mean square and times ``gain``. ``own=False``: the layer projects queries only and reads the keys and values of the layer
+    its cache entry names."""
+
+    def __init__(self, layer_idx: int, spec, eps: float, w_in: torch.Tensor, freq: Optional[torch.Tensor], lam: float,
+                 gain: float, w_o: torch.Tensor, own: bool = True, rot_gain: float = 1.0):
+        self.i = layer_idx
+        self.spec = spec
+        self.eps = eps
+        self.w_in = w_in    # [2 H dim (+ 2 G dim + G vdim), D]: q (| k | v)
+        self.freq = freq    # float64 [rot_dims / 2] or None
+        self.diff = hy.DiffMaps(lam, eps, gain)
+        self.own, self.rot_gain = own, rot_gain
+        self.w_o, self.o_bias = w_o, None  # [D, H vdim]
+        self.head, self.width = spec.vdim, spec.heads * spec.vdim
+
+    def features(self, proj: torch.Tensor, ctx: StepContext, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        sp = self.spec
+        kc, vc = ctx.cache.layer(self.i)
+        q, _ = hy.qkv_prep(proj, None, None, None, self.eps, ctx.positions, ctx.slot0, ctx.b, ctx.s, sp.heads, sp.kv_heads,
+                           sp.dim, sp.vdim, kc if self.own else None, vc if self.own else None, self.freq, maps=2,
+                           rot_gain=self.rot_gain)
+        return hy.attn_bias(q, kc, vc, ctx.slot0, sp.scale, out=out, diff=self.diff)
+
+
+class SharedExpertMoE:
+    """Mixture of gated experts ``W_down (silu(W_gate h) * W_up h)``: router logits with a bias, the ``top`` largest chosen,
+    weights the softmax over the chosen logits, applied to the experts' OUTPUTS; an optional shared expert of the same form
+    runs for every token. The shared expert's gate / up rows and the router's rows read the same input and are one matrix
+    (``[2 ff_shared + E (+ padding to whole 16-row tiles), D]``): a prompt runs them as one product."""
+
+    RULE = hy.RouterRule(normalise=True)
+
+    def __init__(self, experts: int, top: int, w_router: torch.Tensor, router_bias: torch.Tensor, w_gu: torch.Tensor,
+                 w_down: torch.Tensor, shared_gu: Optional[torch.Tensor] = None,
+                 shared_down: Optional[torch.Tensor] = None):
+        self.experts, self.top = experts, top
+        self.router_bias = router_bias  # fp32 [E]
+        self.w_gu, self.w_down = w_gu, w_down  # [E, 2 ff, D] gate rows then up rows, [E, D, ff]
+        rows = ([shared_gu] if shared_gu is not None else []) + [w_router]
+        self.side_ff = shared_gu.shape[0] // 2 if shared_gu is not None else 0
+        n = sum(r.shape[0] for r in rows)
+        if n % 16:
+            rows.append(torch.zeros(16 - n % 16, w_router.shape[1], dtype=w_router.dtype, device=w_router.device))
+        self.w_side = torch.cat(rows, 0).contiguous()
+        c = 2 * self.side_ff
+        self.shared_gu, self.w_router = self.w_side[:c], self.w_side[c:c + experts]  # (views of it: a few rows run GEMVs)
+        self.shared_down = shared_down  # [D, ff_shared]
+
+    def __call__(self, h: torch.Tensor, ctx: StepContext) -> FFOut:
+        m, ff = h.shape[0], self.side_ff
+        extra = hid = None
+        if hy.one_product(h, self.w_side):
+            zs = hy.linear(h, self.w_side)
+            z = zs[:, 2 * ff:2 * ff + self.experts]
+            if ff:
+                hid = hy.glu_rows(zs, hy.ACT_SWIGLU, torch.empty(m, ff, dtype=h.dtype, device=h.device))
+        else:
+            z = hy.linear(h, self.w_router)
+            if ff:
+                hid = hy.linear_glu(h, self.shared_gu, hy.ACT_SWIGLU, torch.empty(m, ff, dtype=h.dtype, device=h.device))
+        if ff:
+            extra = hy.linear(hid, self.shared_down)
+        y, _, row_w = hy.moe_grouped(h, z, None, self.top, 1, 1, self.w_gu, self.w_down, hy.ACT_SWIGLU, self.RULE,
+                                     self.router_bias)
+        return FFOut(y, self.top, extra, row_w=row_w)
+
+
+class SandwichChainBlock:
+    """``x += post1 * rms(mixer(pre1 * rms(x)))``, ``x += post2 * rms(ff(pre2 * rms(x)))`` (gains fp32; a constant residual
+    factor is folded into the output gains). One elementwise kernel per sublayer takes its result (output bias, the mixture's
+    weighted rows, the shared expert), norms it, adds it to the residual and leaves the next sublayer's normed input in
+    ``ctx.h``, in the type its products read."""
+
+    def __init__(self, mixer, post1: torch.Tensor, mlp: Optional[SharedExpertMoE], pre2: Optional[torch.Tensor],
+                 post2: Optional[torch.Tensor], pre1: torch.Tensor, eps: float):
+        self.mixer, self.pre1, self.post1, self.eps = mixer, pre1, post1, eps
+        self.mlp, self.pre2, self.post2 = mlp, pre2, post2
+        self.next_norm: Optional[torch.Tensor] = None  # gain through which the next layer (or the model's end) reads x
+        self.last = False
+
+    def __call__(self, x: torch.Tensor, ctx: StepContext) -> None:
+        mx = self.mixer
+        # (a prompt whose last token alone is wanted norms that row at the end)
+        after = self.next_norm if not self.last or ctx.every_row else None
+        a = mx.features(hy.linear(ctx.h, mx.w_in), ctx,
+                        torch.empty(x.shape[0], mx.width, dtype=ctx.act_dtype, device=x.device))
+        ctx.h = hy.sandwich_update_(x, hy.linear(a, mx.w_o), self.post1, self.eps, bias=mx.o_bias,
+                                    pre=self.pre2 if self.mlp is not None else after, h_dtype=ctx.act_dtype)
+        if self.mlp is not None:
+            f = self.mlp(ctx.h, ctx)
+            ctx.h = hy.sandwich_update_(x, f.y, self.post2, self.eps, f.nsum, f.row_w, extra=f.extra, pre=after,
+                                        h_dtype=ctx.act_dtype)

@@ -49,12 +49,19 @@ def _fokisun():
     return FokisunConfig, FokisunForCausalLM
 
 
+def _zopupel():
+    from ..config import ZopupelConfig
+    from .zopupel import ZopupelForCausalLM
+    return ZopupelConfig, ZopupelForCausalLM
+
+
 # architecture name (lower case) -> () -> (config class, model class)
 MODEL_REGISTRY: Dict[str, Callable[[], Tuple[type, type]]] = {"llama": _llama, "zavevik": _zavevik,
                                                               "zasevik": _zasevik, "besulix": _besulix,
-                                                              "zifisun": _zifisun, "fokisun": _fokisun}
+                                                              "zifisun": _zifisun, "fokisun": _fokisun,
+                                                              "zopupel": _zopupel}
 # families on the layer-list step function (models/layer_list.py): both number formats, the hybrid extension
-LAYER_LIST_FAMILIES = ("zavevik", "zasevik", "besulix", "zifisun", "fokisun")
+LAYER_LIST_FAMILIES = ("zavevik", "zasevik", "besulix", "zifisun", "fokisun", "zopupel")
 
 
 def register(name: str, factory: Callable[[], Tuple[type, type]]) -> None:

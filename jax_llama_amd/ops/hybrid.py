@@ -37,7 +37,12 @@ Mechanisms (each with its constants as arguments, usable by any model of the reg
     forget gate also decides what is written (``lin_scan`` mode 2);
   * ``squash_rows`` / ``depth_update_``: a statistics-free norm (``tanh(alpha x) w + b``) and the residual step of a stack
     whose layers read a weighted sum of every earlier layer's result; ``linear_glu``: gated feed-forward halves written
-    into a column slice, so that several sublayers' features share one output product.
+    into a column slice, so that several sublayers' features share one output product;
+  * ``attn_bias(diff=DiffMaps(...))`` + ``qkv_prep(maps=2)``: differential heads (two softmax maps over the same values, their
+    weighted difference RMS-normed per head); ``qkv_prep(v_is_k=, rot_gain=)`` and queries only: values that are the key
+    columns as projected, a factor on cosine and sine (``yarn_freqs``), layers that read another layer's cache;
+    ``route_grouped(z_bias=)``: a bias on the router's logits; ``sandwich_update_``: the residual step of a stack with norms
+    on both sides of every sublayer, with the next sublayer's input norm.
 """
 from __future__ import annotations
 
@@ -156,6 +161,12 @@ def _use_packed_gemm(x: torch.Tensor, w: torch.Tensor) -> bool:
     return core_available()
 
 
+def one_product(x: torch.Tensor, w: torch.Tensor) -> bool:
+    """Whether matrices that read the same rows ``x`` and lie stacked in ``w`` are better run as one product: a prompt-sized
+    batch on the packed GEMM (whose epilogue has no activation anyway)."""
+    return _gpu(x) and _use_packed_gemm(x, w)
+
+
 class RmsInput:
     """A sublayer's input ``rms_norm(x) * gain`` that is only written out when a consumer needs it in memory: the GEMV
     kernels norm the row they read themselves (``linear`` / ``moe_routed`` take this object in place of a tensor), the
@@ -251,6 +262,16 @@ def prompt_bf16(m: int, cols: int, wdtype) -> bool:
     return wdtype == BF16 and m >= PACKED_GEMM_MIN_M and cols % 8 == 0
 
 
+def glu_rows(gu: torch.Tensor, act: int, out: torch.Tensor, limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
+    """``out [M, F] = act(gu[:, :F], gu[:, F:2F])`` for a gated activation and a product ``gu [M, >= 2F]`` (fp32; more columns
+    may follow); ``out`` fp32 or bf16, maybe a column slice."""
+    f = out.shape[1]
+    if not _gpu(gu):
+        return out.copy_(_act_cpu(gu[:, :2 * f].float(), act, limit, alpha))
+    ext().glu_rows(gu, out, int(act), float(limit), float(alpha))
+    return out
+
+
 def linear_glu(x: torch.Tensor, w: torch.Tensor, act: int, out: torch.Tensor, limit: float = 0.0,
                alpha: float = 1.0) -> torch.Tensor:
     """``out [M, F] = act(x @ w[:F]^T, x @ w[F:]^T)`` for a gated activation; ``out`` may be a column slice of a wider
@@ -261,9 +282,7 @@ def linear_glu(x: torch.Tensor, w: torch.Tensor, act: int, out: torch.Tensor, li
         return out.copy_(_act_cpu(_round_like(x, w) @ w.float().t(), act, limit, alpha))
     if _use_packed_gemm(x, w):
         from . import linear as packed_linear
-        ext().glu_rows(packed_linear(_bf16_rows(x), _packed_weight(w), out_dtype=F32), out, int(act), float(limit),
-                       float(alpha))
-        return out
+        return glu_rows(packed_linear(_bf16_rows(x), _packed_weight(w), out_dtype=F32), act, out, limit, alpha)
     ext().linear_rows(x, None, w, out, None, None, None, x.shape[0], int(act), float(limit), float(alpha), None, None, 0.0)
     return out
 
@@ -516,14 +535,14 @@ SOFTMAX_RULE = RouterRule()
 
 
 def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
-                  rule: RouterRule = SOFTMAX_RULE):
-    """Router over logits ``z [M, E]`` (fp32): scores ``s = softmax(z)`` (or ``sigmoid(z)``); the choice is made on
+                  rule: RouterRule = SOFTMAX_RULE, z_bias: Optional[torch.Tensor] = None):
+    """Router over logits ``z [M, E]`` (fp32, ``+ z_bias [E]`` when given: it counts for choice and weights): scores ``s = softmax(z)`` (or ``sigmoid(z)``); the choice is made on
     ``s + correction`` (``correction [E]``, a selection bias that does not enter the weights); the experts form
     ``groups`` equal groups of neighbours, a group's score is its largest choice score (or its two largest summed), and
     only experts of the ``keep`` best groups can be chosen (ties to the lower index everywhere); the ``top`` largest are
     chosen, weight ``s`` of each, renormalised and scaled as ``rule`` says. Returns ``(row_expert [R], row_w [R])`` in
     (token, choice) order."""
-    zz = z.float()
+    zz = z.float() if z_bias is None else z.float() + z_bias.float()
     m, e_n = zz.shape
     sc = torch.sigmoid(zz) if rule.sigmoid else torch.softmax(zz, -1)
     ch = sc + correction.float().reshape(1, -1) if correction is not None else sc.clone()
@@ -541,7 +560,8 @@ def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int,
 
 
 def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int,
-                w_up: torch.Tensor, w_down: torch.Tensor, act: int = ACT_RELU2, rule: RouterRule = SOFTMAX_RULE):
+                w_up: torch.Tensor, w_down: torch.Tensor, act: int = ACT_RELU2, rule: RouterRule = SOFTMAX_RULE,
+                z_bias: Optional[torch.Tensor] = None):
     """Experts of a ``route_grouped`` mixture: ``z [M, E + I]`` holds the logits of the ``E = w_up.shape[0]`` real
     experts and of ``I`` identity experts behind them (an identity expert returns its input; it has no weights and runs
     no product). ``w_up [E, F, K]``, or for a gated activation ``act`` ``[E, 2F, K]`` (gate rows, then up rows),
@@ -552,7 +572,7 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
     m, e_n, e_all = x.shape[0], w_up.shape[0], z.shape[1]
     r = m * top
     if not _gpu(x):
-        ex, wt = route_grouped(z, correction, top, groups, keep, rule)
+        ex, wt = route_grouped(z, correction, top, groups, keep, rule, z_bias)
         xr = _round_like(x.float(), w_up).repeat_interleave(top, 0)
         y = torch.zeros(r, w_down.shape[1], dtype=F32)
         for e in ex.unique().tolist():
@@ -570,7 +590,7 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
     row_w, sort_w = wts[:r], wts[r:]
     y = torch.empty(r, w_down.shape[1], dtype=F32, device=dev)
     f = w_up.shape[1] // 2 if act_gated(act) else w_up.shape[1]
-    how = (rule.sigmoid, rule.group_top, rule.normalise, rule.scale)
+    how = (rule.sigmoid, rule.group_top, rule.normalise, rule.scale, z_bias)
     if r <= e.GEMV_MAX_R:  # decode: one GEMV per (token, choice) row; rows of identity experts are skipped on the device
         e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, None, None, None, None, *how)
         h = torch.empty(r, f, dtype=F32, device=dev)
@@ -677,6 +697,28 @@ def depth_update_(hist: torch.Tensor, i: int, x: torch.Tensor, x_out: torch.Tens
     ext().depth_update(hist, int(i), bool(store), x, x_out, float(mult), y, bias, ye, int(nsum), row_w, coef,
                        norm.alpha if norm is not None else None, norm.w if norm is not None else None,
                        norm.b if norm is not None else None, h)
+    return h
+
+
+def sandwich_update_(x: torch.Tensor, y: Optional[torch.Tensor], post: Optional[torch.Tensor], eps: float, nsum: int = 1,
+                     row_w: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+                     extra: Optional[torch.Tensor] = None, pre: Optional[torch.Tensor] = None, h_dtype=F32):
+    """The residual step between two sublayers of a stack with an RMS norm on both sides of each, ``x [M, D]`` (fp32, in
+    place): ``x += rms_norm(v) * post`` with ``v[m] = sum_{c < nsum} row_w[m * nsum + c] y[m * nsum + c] (+ bias) (+ extra[m])``
+    (``row_w`` absent: weights 1). ``pre``: also returns the next sublayer's input ``rms_norm(x) * pre`` (fp32 or bf16).
+    ``y`` None: the norm of ``x`` alone."""
+    m, d = x.shape
+    if not _gpu(x):
+        if y is not None:
+            v = y.float().reshape(m, nsum, d)
+            v = (v * row_w.float().reshape(m, nsum, 1) if row_w is not None else v).sum(1)
+            for more in (bias, extra):
+                if more is not None:
+                    v = v + more.float()
+            x.add_(v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * post.float())
+        return rms_rows(x, pre, eps).to(h_dtype) if pre is not None else None
+    h = torch.empty(m, d, dtype=h_dtype, device=x.device) if pre is not None else None
+    ext().sandwich_update(x, y, int(nsum), row_w, bias, extra, post, float(eps), pre, h)
     return h
 
 
@@ -885,12 +927,20 @@ def _expand_index(b: int, t: int, n: int, h: int, device):
     return got
 
 
+class DiffMaps:
+    """Differential heads: two softmax maps per head over the same values, ``a_0`` and ``a_1``; the head's output is
+    ``d / sqrt(mean(d^2) + eps) * gain`` with ``d = a_0 - lam * a_1``."""
+
+    def __init__(self, lam: float, eps: float, gain: float):
+        self.lam, self.eps, self.gain = float(lam), float(eps), float(gain)
+
+
 def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: float, softcap: float = 0.0,
               bias: Optional[torch.Tensor] = None, max_kv: Optional[int] = None,
               sink: Optional[torch.Tensor] = None, chunk: int = 0,
               head_scale: Optional[torch.Tensor] = None, window: int = 0, keep_first: int = 0,
               gate: Optional[torch.Tensor] = None, vdim: Optional[int] = None, gate_cols: bool = False,
-              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+              out: Optional[torch.Tensor] = None, diff: Optional[DiffMaps] = None) -> torch.Tensor:
     """Causal attention of ``q [B, S, H, dim]`` (queries at cache slots ``slot + s``) over ``[B, G, T, .]`` caches:
     ``score = q.k * scale``; ``softcap * tanh(score / softcap)`` if ``softcap > 0``; ``+ bias[min(i - j, last), h]``;
     softmax over ``j <= i``, with ``exp(sink[h])`` added to the denominator when ``sink [H]`` is given (a slot without
@@ -901,9 +951,13 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
     ``keep_first`` slots of a row stay visible to every later query). ``gate [B*S, >= H]`` (a column view is fine): head
     ``h``'s output of token ``m`` is multiplied by ``sigmoid(gate[m, h])``; with ``gate_cols`` (``gate [B*S, >= H*vdim]``) its
     column ``c`` by ``sigmoid(gate[m, h * vdim + c])``. ``kc`` and ``vc`` may be one tensor (latent
-    attention); ``vdim``: the values are the first ``vdim`` columns of ``vc``'s rows. Returns fp32 ``[B*S, H*vdim]``, or
-    ``out``, a column slice of a wider fp32 or bf16 buffer."""
-    b, s, h, dim = q.shape
+    attention); ``vdim``: the values are the first ``vdim`` columns of ``vc``'s rows. ``diff``: differential heads, ``q
+    [B, S, 2 H, dim]`` and ``kc [B, G, T, 2 dim]`` hold the two maps of a head side by side (``sink``, ``head_scale`` and the
+    columns of ``bias`` then count per query head, ``2 h + map``). Returns fp32 ``[B*S, H*vdim]``, or ``out``, a column slice
+    of a wider fp32 or bf16 buffer."""
+    b, s, qh, dim = q.shape
+    maps = 2 if diff is not None else 1
+    h = qh // maps
     g = kc.shape[1]
     vdim = vc.shape[3] if vdim is None else int(vdim)
     if chunk and window:
@@ -911,11 +965,14 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
     if not _gpu(q):
         s0 = _slot_int(slot)
         t = s0 + s
-        k = kc[:, :, :t].float().repeat_interleave(h // g, 1)  # [B, H, t, dim]
+        k = kc[:, :, :t].float().repeat_interleave(h // g, 1)  # [B, H, t, maps * dim]
         v = vc[:, :, :t, :vdim].float().repeat_interleave(h // g, 1)
+        if maps == 2:
+            k = k.unflatten(-1, (maps, dim)).permute(0, 1, 3, 2, 4).reshape(b, qh, t, dim)
+            v = v.repeat_interleave(maps, 1)
         sc = torch.einsum("bshd,bhtd->bhst", q.float(), k) * scale
         if head_scale is not None:
-            sc = sc * head_scale.float().reshape(1, h, 1, 1)
+            sc = sc * head_scale.float().reshape(1, qh, 1, 1)
         if softcap and softcap > 0:
             sc = softcap * torch.tanh(sc / softcap)
         qi = torch.arange(s0, t)[:, None]
@@ -931,11 +988,15 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
             hidden = hidden | ((dist >= window) & (kj >= keep_first))
         sc = sc.masked_fill(hidden[None, None], float("-inf"))
         if sink is not None:
-            sc = torch.cat([sc, sink.float().reshape(1, h, 1, 1).expand(b, h, s, 1)], -1)
+            sc = torch.cat([sc, sink.float().reshape(1, qh, 1, 1).expand(b, qh, s, 1)], -1)
             pr = torch.softmax(sc, -1)[..., :-1]
         else:
             pr = torch.softmax(sc, -1)
         o = torch.einsum("bhst,bhtv->bshv", pr, v)
+        if maps == 2:
+            o = o.unflatten(2, (h, maps))
+            o = o[:, :, :, 0] - diff.lam * o[:, :, :, 1]
+            o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + diff.eps) * diff.gain
         if gate is not None:
             gn = vdim if gate_cols else 1
             o = o * torch.sigmoid(gate[:, :h * gn].float()).reshape(b, s, h, gn)
@@ -948,15 +1009,15 @@ def attn_bias(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, slot, scale: 
     ws, splits, vt = None, 1, None
     if s == 1:
         seen = min(t_cap, chunk) if chunk and chunk > 0 else (min(t_cap, window + keep_first) if window > 0 else t_cap)
-        splits = int(e.attn_decode_splits(b, h, seen))
-        ws = torch.empty(b * h * splits * (vdim + 2), dtype=F32, device=q.device)
+        splits = int(e.attn_decode_splits(b, qh, seen))
+        ws = torch.empty(b * qh * splits * (vdim + 2), dtype=F32, device=q.device)
     elif MMA_PREFILL:
         nb = int(e.attn_prefill_ws_bytes(b, s, g, dim, vdim, kc.shape[2], kc.dtype == BF16)) if vdim == vc.shape[3] else 0
         if nb:  # bf16 caches at the MFMA shapes: the flash kernel over a transposed copy of the values
             vt = torch.empty(nb // 2, dtype=BF16, device=q.device)
     e.attn_bias(q.contiguous(), kc, vc, _slot_tensor(slot, q.device), float(scale), float(softcap or 0.0), bias, out,
                 t_cap, ws, splits, vt, sink, int(chunk or 0), head_scale, int(window or 0), int(keep_first or 0), gate,
-                vdim, bool(gate_cols))
+                vdim, bool(gate_cols), maps, *((diff.lam, diff.eps, diff.gain) if diff is not None else ()))
     return out
 
 
@@ -1067,6 +1128,23 @@ def rotary_freqs(base: float, dims: int, device) -> torch.Tensor:
     return torch.tensor([float(base) ** (-2.0 * i / dims) for i in range(dims // 2)], dtype=torch.float64, device=device)
 
 
+def yarn_freqs(base: float, dims: int, factor: float, original: float, fast: float, slow: float,
+               device) -> Tuple[torch.Tensor, float]:
+    """``(float64 [dims / 2], gain)``: rotary frequencies for contexts ``factor`` times the ``original`` length. Pair ``i``
+    keeps its frequency below the pair that makes ``fast`` full turns over the original length, has it divided by ``factor``
+    past the pair that makes ``slow`` turns, and goes linearly from one to the other between them (the bounds rounded
+    outwards and kept inside the head's rotated part); ``gain = 0.1 ln(factor) + 1`` multiplies every cosine and sine."""
+    freq = rotary_freqs(base, dims, device)
+
+    def pair(turns: float) -> float:
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(pair(fast)), 0), min(math.ceil(pair(slow)), dims - 1)
+    i = torch.arange(dims // 2, dtype=torch.float64, device=device)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
 def _turn_cpu(x: torch.Tensor, pos: torch.Tensor, freq: torch.Tensor, sign: float = 1.0) -> torch.Tensor:
     """Rotate the first ``2 len(freq)`` numbers of the last axis of ``x [M, heads, n]`` by ``sign * pos[m]``: number
     ``i`` pairs with ``i + len(freq)``."""
@@ -1123,20 +1201,26 @@ def rope_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], positions: torch
 
 def qkv_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], q_w: Optional[torch.Tensor], k_w: Optional[torch.Tensor],
              eps: float, positions: torch.Tensor, slot, b: int, s: int, heads: int, kv_heads: int, dim: int, vdim: int,
-             kc: torch.Tensor, vc: torch.Tensor, freq: Optional[torch.Tensor], interleaved: bool = False,
-             v_prev: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None, keep_v: bool = False):
+             kc: Optional[torch.Tensor], vc: Optional[torch.Tensor], freq: Optional[torch.Tensor],
+             interleaved: bool = False, v_prev: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None,
+             keep_v: bool = False, maps: int = 1, v_is_k: bool = False, rot_gain: float = 1.0):
     """From the fused projection ``proj [B*S, H*dim + G*dim + G*vdim (+ more)]`` (+ ``bias``, one number per q / k / v
     column): q divided by the root mean square of ALL its columns, times ``q_w [H*dim]`` (None: no norm), k likewise with
     ``k_w [G*dim]``; then every q / k head rotated by the token's position on its first ``2 len(freq)`` numbers (pairs
     ``2i``, ``2i + 1`` when ``interleaved``, else ``i``, ``i + len(freq)``; None: no rotation). ``v_prev [B*S, G*vdim]``: v
     becomes ``(1 - lam) v + lam v_prev`` (``lam``: one fp32 number). k / v are written into the caches ``[B, G, T, .]`` at
-    ``slot + s``. Returns ``(q [B, S, H, dim] fp32, v)``: ``v [B*S, G*vdim]`` the values before their rounding when ``keep_v``,
-    else None."""
+    ``slot + s``. ``maps = 2``: every head of q and k holds two parts of ``dim`` numbers, each rotated by itself (a key row
+    keeps them side by side). ``v_is_k``: the projection has no value columns, the values are the key columns as projected
+    (with their bias, before norm and rotation). ``rot_gain`` multiplies cosine and sine (the numbers that are not rotated
+    pass). ``kc`` None: ``proj`` holds queries only and nothing is cached. Returns ``(q [B, S, H*maps, dim] fp32, v)``:
+    ``v [B*S, G*vdim]`` the values before their rounding when ``keep_v``, else None."""
     m = b * s
-    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    own = kc is not None
+    heads, kvh = heads * maps, (kv_heads * maps if own else 0)  # dim-sized parts
+    nq, nk, nv = heads * dim, kvh * dim, (kv_heads * vdim if own else 0)
     if not _gpu(proj):
         s0 = _slot_int(slot)
-        y = proj[:, :nq + nk + nv].float()
+        y = proj[:, :nq + nk + (0 if v_is_k else nv)].float()
         if bias is not None:
             y = y + bias.float()
 
@@ -1147,21 +1231,25 @@ def qkv_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], q_w: Optional[tor
             x = x.reshape(m, h, dim)
             if freq is not None:
                 x = (_turn_pairs_cpu if interleaved else _turn_cpu)(x, positions.reshape(-1), freq)
+                x = torch.cat([x[..., :2 * freq.numel()] * rot_gain, x[..., 2 * freq.numel():]], -1)
             return x
 
-        q, k = part(0, nq, q_w, heads), part(nq, nk, k_w, kv_heads)
-        v = y[:, nq + nk:]
+        q = part(0, nq, q_w, heads)
+        if not own:
+            return q.reshape(b, s, heads, dim).contiguous(), None
+        k = part(nq, nk, k_w, kvh)
+        v = y[:, nq:nq + nk] if v_is_k else y[:, nq + nk:]
         if v_prev is not None:
             v = (1.0 - lam.float()) * v + lam.float() * v_prev.float()
-        kc[:, :, s0:s0 + s] = k.reshape(b, s, kv_heads, dim).permute(0, 2, 1, 3).to(kc.dtype)
+        kc[:, :, s0:s0 + s] = k.reshape(b, s, kv_heads, maps * dim).permute(0, 2, 1, 3).to(kc.dtype)
         vc[:, :, s0:s0 + s] = v.reshape(b, s, kv_heads, vdim).permute(0, 2, 1, 3).to(vc.dtype)
         return q.reshape(b, s, heads, dim).contiguous(), v.contiguous() if keep_v else None
     dev = proj.device
     q = torch.empty(b, s, heads, dim, dtype=F32, device=dev)
     v = torch.empty(m, nv, dtype=F32, device=dev) if keep_v else None
     ext().qkv_prep(proj, bias, q_w, k_w, float(eps), positions.reshape(-1).to(torch.int32).contiguous(),
-                   _slot_tensor(slot, dev), b, s, heads, kv_heads, dim, vdim, kc, vc, q, freq, not interleaved, v_prev,
-                   lam if v_prev is not None else None, v)
+                   _slot_tensor(slot, dev), b, s, heads // maps, kv_heads, dim, vdim, kc, vc, q, freq, not interleaved,
+                   v_prev, lam if v_prev is not None else None, v, maps, bool(v_is_k), float(rot_gain))
     return q, v
 
 
