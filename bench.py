@@ -90,6 +90,9 @@ def main():
     ap.add_argument("--depth-compare", action="store_true", help="the same comparison for the family that averages over its "
                     "depth (rotary, latent and running-memory layers, mixer and feed-forward side by side): Fokisun beside "
                     "Zifisun (the closest family), Besulix (the closest recurrence) and LLaMA")
+    ap.add_argument("--sandwich-compare", action="store_true", help="the same comparison for the family of differential "
+                    "attention and attention whose values are its keys, norms on both sides of every sublayer: Zopupel beside "
+                    "Fokisun (the closest family), Zasevik (the other with such norms) and LLaMA")
     ap.add_argument("--hybrid-sizes", nargs="*", default=["2k", "4k"])
     ap.add_argument("--hybrid-families", nargs="*", default=["zavevik", "llama"])
     ap.add_argument("--hybrid-batches", type=int, nargs="*", default=[1, 8])
@@ -102,6 +105,9 @@ def main():
         return _hybrid_compare(args)
     if args.depth_compare:
         args.hybrid_families = ["fokisun", "zifisun", "besulix", "llama"]
+        return _hybrid_compare(args)
+    if args.sandwich_compare:
+        args.hybrid_families = ["zopupel", "fokisun", "zasevik", "llama"]
         return _hybrid_compare(args)
     if args.recurrent_compare:
         args.hybrid_families = ["besulix", "zavevik", "llama"]

@@ -521,29 +521,39 @@ __global__ void __launch_bounds__(64 * AB_MAX_VREG) attn_diff_merge_kernel(AttnB
   __shared__ float red[AB_MAX_VREG];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.x, b = blockIdx.y, waves = blockDim.x >> 6;
   const int c = min((int)threadIdx.x, p.vdim - 1);
-  float o = 0.f;
+  const float* w = p.ws + ((size_t)b * p.H + h) * 2 * p.splits * (p.vdim + 2);
+  const size_t next = (size_t)p.splits * (p.vdim + 2);  // from a head's first map to its second
+  float ms[2] = {-INFINITY, -INFINITY}, ls[2] = {0.f, 0.f}, wt[2], l[2], a[2] = {0.f, 0.f}, part[2][32];
 #pragma unroll
   for (int map = 0; map < 2; ++map) {
-    const float* w = p.ws + (((size_t)b * p.H + h) * 2 + map) * p.splits * (p.vdim + 2);
-    float ms = -INFINITY, ls = 0.f;
     if (lane < p.splits) {
-      ms = w[(size_t)lane * (p.vdim + 2)];
-      ls = w[(size_t)lane * (p.vdim + 2) + 1];
+      ms[map] = w[map * next + (size_t)lane * (p.vdim + 2)];
+      ls[map] = w[map * next + (size_t)lane * (p.vdim + 2) + 1];
     }
-    float part[64];
-#pragma unroll
-    for (int sp = 0; sp < 64; ++sp) part[sp] = w[(size_t)min(sp, p.splits - 1) * (p.vdim + 2) + 2 + c];
-    const float m = wave_max(ls > 0.f ? ms : -INFINITY);
-    const float wt = ls > 0.f ? expf(ms - m) : 0.f;
-    const float l = wave_sum(ls * wt);
-    float a = 0.f;
-#pragma unroll
-    for (int sp = 0; sp < 64; ++sp) {
-      const float ws = __shfl(wt, sp, 64);
-      a = fmaf(part[sp], sp < p.splits ? ws : 0.f, a);
-    }
-    o = fmaf(map ? -p.diff_lambda : 1.f, a / l, o);
   }
+  for (int s0 = 0; s0 < p.splits; s0 += 32) {  // 32 splits of both maps per round trip, the first beside the maxima
+#pragma unroll
+    for (int map = 0; map < 2; ++map)
+#pragma unroll
+      for (int sp = 0; sp < 32; ++sp)
+        part[map][sp] = w[map * next + (size_t)min(s0 + sp, p.splits - 1) * (p.vdim + 2) + 2 + c];
+    if (s0 == 0) {
+#pragma unroll
+      for (int map = 0; map < 2; ++map) {
+        const float m = wave_max(ls[map] > 0.f ? ms[map] : -INFINITY);
+        wt[map] = ls[map] > 0.f ? expf(ms[map] - m) : 0.f;
+        l[map] = wave_sum(ls[map] * wt[map]);
+      }
+    }
+#pragma unroll
+    for (int map = 0; map < 2; ++map)
+#pragma unroll
+      for (int sp = 0; sp < 32; ++sp) {  // (a split without keys holds zeros and has weight 0; lanes past the splits: 0)
+        const float ws = __shfl(wt[map], s0 + sp, 64);
+        a[map] = fmaf(part[map][sp], ws, a[map]);
+      }
+  }
+  const float o = a[0] / l[0] - p.diff_lambda * (a[1] / l[1]);
   const bool on = (int)threadIdx.x < p.vdim;
   float ss = wave_sum(on ? o * o : 0.f);
   if (lane == 0) red[wave] = ss;

@@ -75,9 +75,9 @@ void embed_rows(Tensor ids, Tensor table, int64_t col0, Tensor out, double scale
      "embed_rows");
 }
 
-void linear_rows(Tensor a, OptT a_idx, Tensor w, Tensor out, OptT dst_idx, OptT offs, OptT row_expert, int64_t R,
-                 int64_t act, double act_limit, double act_alpha, OptT a_scale, OptT a_norm_w, double a_norm_eps,
-                 int64_t even_rows, bool add_out) {
+jla::RowLinear row_linear(Tensor a, OptT a_idx, Tensor w, Tensor out, OptT dst_idx, OptT offs, OptT row_expert, int64_t R,
+                          int64_t act, double act_limit, double act_alpha, OptT a_scale, OptT a_norm_w, double a_norm_eps,
+                          int64_t even_rows, bool add_out) {
   jla::RowLinear p{};
   p.even_rows = even_rows;
   p.add_out = add_out;
@@ -115,7 +115,21 @@ void linear_rows(Tensor a, OptT a_idx, Tensor w, Tensor out, OptT dst_idx, OptT 
     p.a_norm_eps = a_norm_eps;
   }
   check(p.E == 1 || p.offs || p.row_expert, "linear_rows: stacked experts need offs or row_expert");
-  rc(jla::hy_linear_rows(p, stream()), "linear_rows");
+  return p;
+}
+
+void linear_rows(Tensor a, OptT a_idx, Tensor w, Tensor out, OptT dst_idx, OptT offs, OptT row_expert, int64_t R,
+                 int64_t act, double act_limit, double act_alpha, OptT a_scale, OptT a_norm_w, double a_norm_eps,
+                 int64_t even_rows, bool add_out) {
+  rc(jla::hy_linear_rows(row_linear(a, a_idx, w, out, dst_idx, offs, row_expert, R, act, act_limit, act_alpha, a_scale, a_norm_w,
+                                    a_norm_eps, even_rows, add_out),
+                         stream()),
+     "linear_rows");
+}
+
+// p and q from row_linear: the tensors they were made from must be alive
+void linear_rows_pair(const jla::RowLinear& p, const jla::RowLinear& q) {
+  rc(jla::hy_linear_rows_pair(p, q, stream()), "linear_rows_pair");
 }
 
 // whether a dense linear of `rows` rows with `n` output columns runs the GEMV (where an input norm can be fused)
@@ -845,6 +859,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("offs"), py::arg("row_expert"), py::arg("R"), py::arg("act"), py::arg("act_limit"), py::arg("act_alpha"),
         py::arg("a_scale"), py::arg("a_norm_w"), py::arg("a_norm_eps"), py::arg("even_rows") = 0,
         py::arg("add_out") = false);
+  py::class_<jla::RowLinear>(m, "RowLinear");
+  m.def("row_linear", &row_linear, py::arg("a"), py::arg("a_idx"), py::arg("w"), py::arg("out"), py::arg("dst_idx"),
+        py::arg("offs"), py::arg("row_expert"), py::arg("R"), py::arg("act"), py::arg("act_limit"), py::arg("act_alpha"),
+        py::arg("a_scale"), py::arg("a_norm_w"), py::arg("a_norm_eps"), py::arg("even_rows") = 0,
+        py::arg("add_out") = false);
+  m.def("linear_rows_pair", &linear_rows_pair);
   m.def("route_table", &route_table);
   m.def("route_topk", &route_topk);
   m.def("dense_is_gemv", &dense_is_gemv);

@@ -61,6 +61,9 @@ inline bool hy_act_gated(int act) {
 // per row group); else the 64 x 64 MFMA tiles (offs: expert-grouped).
 constexpr int HY_GEMV_MAX_R = 8;
 int hy_linear_rows(const RowLinear& p, hipStream_t s);
+// two independent linears; one launch where both run the GEMV with the same kind of epilogue (gated or not) at the row counts
+// of a mixture's experts (p) beside its shared expert (q), else one after the other
+int hy_linear_rows_pair(const RowLinear& p, const RowLinear& q, hipStream_t s);
 
 // Table routing: expert of (token m, choice c) = table[ids[m], c]. Writes row_expert[R] and row_tok[R] in (m, c) order
 // (R = M * top), and the expert-sorted order: sort_tok[p] (token of sorted row p), sort_dst[p] (its (m, c) row),

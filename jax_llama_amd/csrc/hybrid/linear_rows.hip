@@ -225,19 +225,19 @@ JLA_DEV float lr_round(float v, const float*) { return v; }
 // together; inside `if (row < rows)` branches each step waits for its own loads. The 8-row form keeps the branches:
 // without them it holds too many registers to keep the chip occupied (measured slower, 1.0 -> 1.36 ms on an 8-row step).
 template <typename WT, int SWIGLU, int LR_CPW, int NORM, int NRT>
-__global__ void __launch_bounds__(LR_THREADS) lr_gemv_kernel(RowLinear p, int rows_per_group) {
+JLA_DEV void lr_gemv_block(const RowLinear& p, int rows_per_group, int bx, int by) {
   constexpr int MAXR = NRT;
   // 512-column steps whose loads go out together: fewer where a step already holds many rows x columns in registers
   constexpr bool GUARD = NRT == 8;
   constexpr int LR_WORK = NRT * LR_CPW * (SWIGLU ? 2 : 1);
   constexpr int LR_UNR = GUARD ? 4 : (LR_WORK >= 16 ? 1 : (LR_WORK >= 8 ? 2 : 4));
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int n0 = (blockIdx.x * (LR_THREADS / 64) + wave) * LR_CPW;
+  const int n0 = (bx * (LR_THREADS / 64) + wave) * LR_CPW;
   if (n0 >= p.N) return;
-  // rows of this group: a fixed count, one row with its own expert, or (offs) every row of expert blockIdx.y
-  int g0 = blockIdx.y * rows_per_group, g1 = min(g0 + rows_per_group, p.R), e = 0;
+  // rows of this group: a fixed count, one row with its own expert, or (offs) every row of expert by
+  int g0 = by * rows_per_group, g1 = min(g0 + rows_per_group, p.R), e = 0;
   if (p.offs) {
-    e = blockIdx.y;
+    e = by;
     g0 = p.offs[e];
     g1 = p.offs[e + 1];
   } else if (p.row_expert) {
@@ -334,6 +334,20 @@ __global__ void __launch_bounds__(LR_THREADS) lr_gemv_kernel(RowLinear p, int ro
   }
 }
 
+template <typename WT, int SWIGLU, int LR_CPW, int NORM, int NRT>
+__global__ void __launch_bounds__(LR_THREADS) lr_gemv_kernel(RowLinear p, int rows_per_group) {
+  lr_gemv_block<WT, SWIGLU, LR_CPW, NORM, NRT>(p, rows_per_group, blockIdx.x, blockIdx.y);
+}
+
+// Two independent linears in one launch (a mixture's experts beside its shared expert): the first na workgroups run p, the
+// others q. A decode step's linears are too short to reach the memory's rate one by one.
+template <typename WT, int SWIGLU, int NRA, int NRB>
+__global__ void __launch_bounds__(LR_THREADS) lr_gemv_pair_kernel(RowLinear p, RowLinear q, int na, int gxa, int gxb) {
+  const int id = blockIdx.x;
+  if (id < na) lr_gemv_block<WT, SWIGLU, 1, 0, NRA>(p, NRA, id % gxa, id / gxa);
+  else lr_gemv_block<WT, SWIGLU, 1, 0, NRB>(q, NRB, (id - na) % gxb, (id - na) / gxb);
+}
+
 // rows at or below which an expert-sorted batch runs the expert-grouped GEMV (each expert's weights streamed once)
 constexpr int HY_GROUPED_GEMV_MAX_R = 64;
 // output columns at or below which a dense linear of any row count runs the GEMV
@@ -352,6 +366,57 @@ bool hy_linear_rows_is_gemv(const RowLinear& p) {
   return lr_grouped(p) || lr_skinny(p) || (p.R <= HY_GEMV_MAX_R && (!p.offs || p.row_expert) && lr_fp32_io(p));
 }
 
+// rows per pass of a GEMV: one for per-row experts, the row count rounded up to 2 / 4 / 8 for a dense batch
+// (expert-grouped: 8 per pass over an expert's rows, whose count only the device knows, unless the caller says that every
+// expert has the same few)
+static int lr_pass_rows(const RowLinear& p) {
+  const bool grouped = lr_grouped(p);
+  const int want = p.row_expert && !grouped ? 1 : (grouped ? (p.even_rows > 0 ? p.even_rows : HY_GEMV_MAX_R) : p.R);
+  return want > 4 ? HY_GEMV_MAX_R : (want > 2 ? 4 : (want > 1 ? 2 : 1));
+}
+
+int hy_linear_rows_pair(const RowLinear& p, const RowLinear& q, hipStream_t s) {
+  auto plain = [](const RowLinear& x) {  // what the one-launch form takes
+    return x.R > 0 && x.N > 0 && x.K > 0 && x.lda >= x.K && x.ldo >= x.N && x.E >= 1 && x.E <= 65535 && x.N < 8192 &&
+           !x.a_norm_w && lr_fp32_io(x) && hy_linear_rows_is_gemv(x) && x.act >= HY_ACT_NONE && x.act <= HY_ACT_GELU_GLU &&
+           x.act != HY_ACT_SOFTCAP;
+  };
+  const bool gated = hy_act_gated(p.act);
+  const int ra = lr_pass_rows(p), rb = lr_pass_rows(q);  // instances: per-row experts beside 1, 2 or 4 rows; 8 beside 8
+  if (!plain(p) || !plain(q) || p.wbf16 != q.wbf16 || gated != hy_act_gated(q.act) ||
+      !((ra == 1 && rb <= 4) || (ra == 8 && rb == 8))) {
+    const int r = hy_linear_rows(p, s);
+    return r ? r : hy_linear_rows(q, s);
+  }
+  RowLinear a = p, b = q;
+  if (!lr_grouped(p)) a.offs = nullptr;
+  if (!lr_grouped(q)) b.offs = nullptr;
+  auto groups = [](const RowLinear& x, int nrt) { return x.offs ? x.E : (x.R + nrt - 1) / nrt; };
+  const int gxa = (a.N + 3) / 4, gxb = (b.N + 3) / 4;
+  const long long na = (long long)gxa * groups(a, ra), nb = (long long)gxb * groups(b, rb);
+  if (na + nb > 0x7fffffffLL) return -4;
+#define LR_PAIR_N(WT, SW, NRA, NRB) \
+  lr_gemv_pair_kernel<WT, SW, NRA, NRB><<<(unsigned)(na + nb), LR_THREADS, 0, s>>>(a, b, (int)na, gxa, gxb)
+#define LR_PAIR(WT, SW)                        \
+  do {                                         \
+    if (ra == 8) LR_PAIR_N(WT, SW, 8, 8);      \
+    else if (rb == 1) LR_PAIR_N(WT, SW, 1, 1); \
+    else if (rb == 2) LR_PAIR_N(WT, SW, 1, 2); \
+    else LR_PAIR_N(WT, SW, 1, 4);              \
+  } while (0)
+  if (p.wbf16) {
+    if (gated) LR_PAIR(bf16_t, 1);
+    else LR_PAIR(bf16_t, 0);
+  } else {
+    if (gated) LR_PAIR(float, 1);
+    else LR_PAIR(float, 0);
+  }
+#undef LR_PAIR
+#undef LR_PAIR_N
+  JLA_CHECK_LAUNCH();
+  return 0;
+}
+
 int hy_linear_rows(const RowLinear& p, hipStream_t s) {
   if (p.R < 0 || p.N <= 0 || p.K <= 0 || p.lda < p.K || p.ldo < p.N || p.E < 1) return -1;
   if (p.act < HY_ACT_NONE || p.act > HY_ACT_GELU_GLU) return -8;
@@ -366,11 +431,7 @@ int hy_linear_rows(const RowLinear& p, hipStream_t s) {
   if (p.a_norm_w && (!small || p.a_bf16)) return -10;  // (the tiles take a normed activation, they do not norm it)
   if (small) {
     if (p.a_bf16 || p.out_bf16) return -7;  // (the GEMV reads and writes fp32)
-    // rows per pass: one for per-row experts, the row count rounded up to 2 / 4 / 8 for a dense batch
-    // (expert-grouped: 8 per pass over an expert's rows, whose count only the device knows, unless the caller says that
-    // every expert has the same few)
-    const int want = p.row_expert && !grouped ? 1 : (grouped ? (p.even_rows > 0 ? p.even_rows : HY_GEMV_MAX_R) : p.R);
-    const int nrt = want > 4 ? HY_GEMV_MAX_R : (want > 2 ? 4 : (want > 1 ? 2 : 1));
+    const int nrt = lr_pass_rows(p);
     const int rpg = nrt;
     if (p.a_norm_w && nrt > 2) return -11;  // (the norm-fusing instances exist for one and two rows)
     const int cpw = p.N >= 8192 ? 4 : 1;

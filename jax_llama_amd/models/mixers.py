@@ -825,18 +825,19 @@ class SharedExpertMoE:
 
     def __call__(self, h: torch.Tensor, ctx: StepContext) -> FFOut:
         m, ff = h.shape[0], self.side_ff
-        extra = hid = None
-        if hy.one_product(h, self.w_side):
+        extra = None
+        if hy.one_product(h, self.w_side):  # a prompt: one product for the shared expert's first half and the router
             zs = hy.linear(h, self.w_side)
             z = zs[:, 2 * ff:2 * ff + self.experts]
             if ff:
-                hid = hy.glu_rows(zs, hy.ACT_SWIGLU, torch.empty(m, ff, dtype=h.dtype, device=h.device))
+                hid = torch.empty(m, ff, dtype=h.dtype, device=h.device)
+                extra = hy.linear(hy.glu_rows(zs, hy.ACT_SWIGLU, hid), self.shared_down)
         else:
             z = hy.linear(h, self.w_router)
-            if ff:
-                hid = hy.linear_glu(h, self.shared_gu, hy.ACT_SWIGLU, torch.empty(m, ff, dtype=h.dtype, device=h.device))
-        if ff:
-            extra = hy.linear(hid, self.shared_down)
+            if ff:  # a few rows: the shared expert runs beside the routed ones
+                y, _, row_w, extra = hy.moe_grouped_shared(h, z, self.top, self.w_gu, self.w_down, self.shared_gu,
+                                                           self.shared_down, hy.ACT_SWIGLU, self.RULE, self.router_bias)
+                return FFOut(y, self.top, extra, row_w=row_w)
         y, _, row_w = hy.moe_grouped(h, z, None, self.top, 1, 1, self.w_gu, self.w_down, hy.ACT_SWIGLU, self.RULE,
                                      self.router_bias)
         return FFOut(y, self.top, extra, row_w=row_w)

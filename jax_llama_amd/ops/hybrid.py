@@ -569,6 +569,19 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
     ``(y [M * top, D], row_expert [M * top], row_w [M * top])`` in (token, choice) order: ``y`` rows of real experts hold
     ``W_down act(W_up x)`` unweighted, rows whose expert is ``>= E`` hold nothing (the caller's ``hc_update_`` puts the
     weighted sum together)."""
+    return _moe_grouped(x, z, correction, top, groups, keep, w_up, w_down, act, rule, z_bias, None)[:3]
+
+
+def moe_grouped_shared(x: torch.Tensor, z: torch.Tensor, top: int, w_up: torch.Tensor, w_down: torch.Tensor,
+                       shared_up: torch.Tensor, shared_down: torch.Tensor, act: int, rule: RouterRule = SOFTMAX_RULE,
+                       z_bias: Optional[torch.Tensor] = None):
+    """``moe_grouped`` (one group) and a shared expert of the same form side by side: ``(y, row_expert, row_w, extra)`` with
+    ``extra [M, D] = shared_down act(shared_up x)``. The experts' and the shared expert's products of a few rows run in one
+    launch each."""
+    return _moe_grouped(x, z, None, top, 1, 1, w_up, w_down, act, rule, z_bias, (shared_up, shared_down))
+
+
+def _moe_grouped(x, z, correction, top, groups, keep, w_up, w_down, act, rule, z_bias, shared):
     m, e_n, e_all = x.shape[0], w_up.shape[0], z.shape[1]
     r = m * top
     if not _gpu(x):
@@ -581,7 +594,10 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
             sel = (ex == e).nonzero().squeeze(1)
             hid = _act_cpu(xr[sel] @ w_up[e].float().t(), act, 0.0, 1.0)
             y[sel] = _round_like(hid, w_down) @ w_down[e].float().t()
-        return y, ex.to(torch.int32), wt
+        extra = None
+        if shared is not None:
+            extra = linear(linear(x.float(), shared[0], act=act), shared[1])
+        return y, ex.to(torch.int32), wt, extra
     dev = x.device
     e = ext()
     idx = torch.empty(4 * r + e_all + 1, dtype=torch.int32, device=dev)
@@ -594,8 +610,8 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
     if r <= e.GEMV_MAX_R:  # decode: one GEMV per (token, choice) row; rows of identity experts are skipped on the device
         e.route_grouped(z, correction, e_all, top, groups, keep, row_expert, row_tok, row_w, None, None, None, None, *how)
         h = torch.empty(r, f, dtype=F32, device=dev)
-        e.linear_rows(x, row_tok, w_up, h, None, None, row_expert, r, int(act), 0.0, 1.0, None, None, 0.0)
-        e.linear_rows(h, None, w_down, y, None, None, row_expert, r, ACT_NONE, 0.0, 1.0, None, None, 0.0)
+        up = (x, row_tok, w_up, h, None, None, row_expert, r, int(act), 0.0, 1.0, None, None, 0.0)
+        down = (h, None, w_down, y, None, None, row_expert, r, ACT_NONE, 0.0, 1.0, None, None, 0.0)
     else:
         # expert-grouped over the sorted rows; identity experts sort behind the real ones, past the last offset the
         # linears look at
@@ -609,9 +625,20 @@ def moe_grouped(x: torch.Tensor, z: torch.Tensor, correction: Optional[torch.Ten
         if keep_bf16 and x.dtype == F32 and x.is_contiguous() and x.numel() % 8 == 0:
             xa = torch.empty(x.shape, dtype=BF16, device=dev)
             e.cast_bf16(x, xa)
-        e.linear_rows(xa, sort_tok, w_up, h, None, offs, None, r, int(act), 0.0, 1.0, None, None, 0.0)
-        e.linear_rows(h, None, w_down, y, sort_dst, offs, None, r, ACT_NONE, 0.0, 1.0, None, None, 0.0)
-    return y, row_expert, row_w
+        up = (xa, sort_tok, w_up, h, None, offs, None, r, int(act), 0.0, 1.0, None, None, 0.0)
+        down = (h, None, w_down, y, sort_dst, offs, None, r, ACT_NONE, 0.0, 1.0, None, None, 0.0)
+    if shared is None:
+        e.linear_rows(*up)
+        e.linear_rows(*down)
+        return y, row_expert, row_w, None
+    fs = shared[1].shape[1]
+    hs = torch.empty(m, fs, dtype=x.dtype, device=dev)
+    extra = torch.empty(m, shared[1].shape[0], dtype=F32, device=dev)
+    e.linear_rows_pair(e.row_linear(*up),
+                       e.row_linear(x, None, shared[0], hs, None, None, None, m, int(act), 0.0, 1.0, None, None, 0.0))
+    e.linear_rows_pair(e.row_linear(*down),
+                       e.row_linear(hs, None, shared[1], extra, None, None, None, m, ACT_NONE, 0.0, 1.0, None, None, 0.0))
+    return y, row_expert, row_w, extra
 
 
 def hc_in(xs: torch.Tensor, a: torch.Tensor) -> torch.Tensor:

@@ -336,10 +336,32 @@ def fokisun_like(width: int, heads: int, kv_heads: int, head_dim: int, ffn: int,
                                     "residual_mult": 0.5, "logit_scale": 0.5, "layers": [turn[i % 4] for i in range(layers)]})
 
 
+def zopupel_like(width: int, heads: int, kv_heads: int, head_dim: int, ffn: int, layers: int, vocab: int,
+                 experts: int = 8, top: int = 2):
+    """A Zopupel config whose layers have a LLaMA layer's sizes, in turn: attention whose values are its keys (``heads`` /
+    ``kv_heads`` heads of ``head_dim``, all of it rotated, YaRN by 4 from 512 positions), differential attention (``heads`` /
+    ``kv_heads`` heads of two maps of ``head_dim / 2`` and values of ``head_dim``), the first kind again, and differential
+    attention on the second layer's keys and values; each with ``top`` of ``experts`` experts of ``ffn / 4`` plus a shared
+    expert of ``ffn / 2`` (the active width of the dense FFN at top 2)."""
+    from ..config import ZopupelConfig
+    half = head_dim // 2
+    kva = dict(heads=heads, kv_heads=kv_heads, dim=head_dim, vdim=head_dim, scale=head_dim ** -0.5,
+               rot={"base": 1e4, "dims": head_dim, "scaling": {"factor": 4.0, "original": 512, "fast": 32.0, "slow": 1.0}})
+    dif = dict(heads=heads, kv_heads=kv_heads, dim=half, vdim=head_dim, scale=half ** -0.5, diff=0.5,
+               rot={"base": 1e4, "dims": half, "scaling": {"factor": 2.0}})
+    moe = {"kind": "moe", "expert": {"ff": ffn // 4}, "shared": {"ff": ffn // 2}, "router": {"experts": experts, "top": top}}
+    ls = []
+    for i in range(layers):
+        ls.append({"type": "attention" if i % 2 else "attention_2", "mlp": moe,
+                   "mixer": kva if i % 2 == 0 else (dict(dif, kv_from=i - 2) if i % 4 == 3 else dif)})
+    return ZopupelConfig.from_dict({"architecture": "Zopupel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                    "residual_mult": 0.5, "layers": ls})
+
+
 def hybrid_compare(device, sizes=("2k", "4k"), prompt_len: int = 2048, gen_len: int = 64, batches=(1, 8),
                    families=("zavevik", "llama"), progress=lambda m: None) -> Dict[str, object]:
-    """Prefill and decode throughput of the layer-list families (Zavevik, Zasevik, Besulix, Zifisun, Fokisun) beside LLaMA at equal
-    layer sizes (random weights, bf16, synthetic ids), all through the decode engine: ``prefill_tokens_per_sec`` of one warm ``prompt_len``-token prompt per row
+    """Prefill and decode throughput of the layer-list families (Zavevik, Zasevik, Besulix, Zifisun, Fokisun, Zopupel) beside LLaMA at
+    equal layer sizes (random weights, bf16, synthetic ids), all through the decode engine: ``prefill_tokens_per_sec`` of one warm ``prompt_len``-token prompt per row
     and hipGraph-replayed ``decode_ms_per_token`` over ``gen_len`` steps behind it."""
     from ..config import LLaMAConfig
     from ..models.llama import LLaMAForCausalLM
@@ -364,6 +386,9 @@ def hybrid_compare(device, sizes=("2k", "4k"), prompt_len: int = 2048, gen_len: 
             elif family == "fokisun":
                 from ..models.fokisun import FokisunForCausalLM
                 model = FokisunForCausalLM(fokisun_like(**sz), device=device, dtype=torch.bfloat16, seed=1)
+            elif family == "zopupel":
+                from ..models.zopupel import ZopupelForCausalLM
+                model = ZopupelForCausalLM(zopupel_like(**sz), device=device, dtype=torch.bfloat16, seed=1)
             else:
                 cfg = LLaMAConfig(vocab_size=sz["vocab"], hidden_size=sz["width"], intermediate_size=sz["ffn"],
                                   num_hidden_layers=sz["layers"], num_attention_heads=sz["heads"],

@@ -331,6 +331,35 @@ def test_attention_windows_gates_and_wide_value_rows(dt, shape, window, keep):
         hy.attn_bias(q, kc, vc, s0, 1.0, chunk=8, window=4)
 
 
+@pytest.mark.parametrize("dt", DTYPES)
+@pytest.mark.parametrize("shape", [  # plain / fast decode, plain / MFMA prefill
+    dict(b=2, s=1, s0=300, h=4, g=2, dim=24, vdim=40), dict(b=1, s=1, s0=4300, h=2, g=1, dim=64, vdim=128),
+    dict(b=2, s=1, s0=129, h=6, g=3, dim=128, vdim=64), dict(b=1, s=1, s0=70, h=1, g=1, dim=8, vdim=500),
+    dict(b=1, s=70, s0=131, h=4, g=2, dim=24, vdim=40), dict(b=2, s=150, s0=77, h=4, g=2, dim=64, vdim=128),
+    dict(b=1, s=33, s0=0, h=2, g=2, dim=128, vdim=64), dict(b=1, s=2, s0=63, h=8, g=1, dim=80, vdim=128)])
+@pytest.mark.parametrize("extras", ["none", "window", "chunk", "sink"])
+def test_differential_heads_in_every_kernel(dt, shape, extras):
+    """Two maps per head over the same values, alone and with the other mechanisms of the attention op (per-map sinks, score
+    factors and distance biases, windows with kept keys, blocks, soft cap, gates per head and per column), in every attention
+    kernel against the CPU op; output into a column slice."""
+    b, s, s0, h, g, dim, vdim = (shape[k] for k in ("b", "s", "s0", "h", "g", "dim", "vdim"))
+    t = s0 + s + 3
+    q = _rand(b, s, 2 * h, dim, std=0.5)
+    kc, vc = _rand(b, g, t, 2 * dim, dt=dt), _rand(b, g, t, vdim, dt=dt)
+    kw = {"none": {}, "window": dict(window=50, keep_first=5, gate=_rand(b * s, h + 2)[:, 1:h + 1]),
+          "chunk": dict(chunk=37, softcap=3.0, bias=_rand(90, 2 * h)),
+          "sink": dict(sink=_rand(2 * h), head_scale=_rand(2 * h), gate=_rand(b * s, h * vdim + 3), gate_cols=True)}[extras]
+    diff = hy.DiffMaps(0.7, 1e-3, 0.6)
+    ref = hy.attn_bias(q, kc, vc, s0, dim ** -0.5, diff=diff, **kw)
+    dev = {k: v.to(DEV) if torch.is_tensor(v) else v for k, v in kw.items()}
+    wide = torch.zeros(b * s, h * vdim + 8, device=DEV)
+    got = hy.attn_bias(q.to(DEV), kc.to(DEV), vc.to(DEV), s0, dim ** -0.5, diff=diff, out=wide[:, 4:4 + h * vdim], **dev)
+    # (the MFMA prefill rounds q to bf16 for the score product like any other matrix operand)
+    mma = dt == torch.bfloat16 and s > 1 and dim in (64, 80, 128) and vdim in (64, 128)
+    _close(got, ref, 5e-2 if mma else 5e-5, f"differential heads, {extras}")
+    assert float(wide[:, :4].abs().max()) == 0.0 and float(wide[:, 4 + h * vdim:].abs().max()) == 0.0
+
+
 @pytest.mark.parametrize("m,e,top,groups,keep", [(1, 10, 2, 5, 3), (7, 1, 1, 1, 1), (40, 12, 4, 4, 2), (300, 64, 5, 8, 3),
                                                  (9, 70, 6, 7, 1), (65, 1000, 8, 10, 4), (33, 20, 4, 4, 3)])
 @pytest.mark.parametrize("biased", [True, False])
@@ -355,6 +384,20 @@ def test_route_grouped(m, e, top, groups, keep, biased):
     assert int(offs[0]) == 0 and int(offs[e]) == r and torch.equal(torch.sort(sdst).values.long(), torch.arange(r))
     assert torch.equal(ex[sdst.long()], torch.sort(ex).values) and torch.equal(stok, tok[sdst.long()])
     _close(wts[r:], wts[:r][sdst.long().to(DEV)], 0.0, "sorted weights")
+
+
+@pytest.mark.parametrize("m,e,top", [(1, 8, 2), (70, 8, 2), (33, 130, 4)])
+def test_router_bias_on_the_logits(m, e, top):
+    """A bias on the logits counts for choice and weights (beside a correction, which counts for the choice alone)."""
+    z, zb, corr = _rand(m, e, std=2.0), _rand(e, std=2.0), _rand(e, std=0.05)
+    d, ff = 16, 8
+    w_up, w_down, x = _rand(e, 2 * ff, d), _rand(e, d, ff), _rand(m, d)
+    rule = hy.RouterRule(normalise=True)
+    a = hy.moe_grouped(x, z, corr, top, 1, 1, w_up, w_down, hy.ACT_SWIGLU, rule, zb)
+    b = hy.moe_grouped(x.to(DEV), z.to(DEV), corr.to(DEV), top, 1, 1, w_up.to(DEV), w_down.to(DEV), hy.ACT_SWIGLU, rule, zb.to(DEV))
+    assert torch.equal(b[1].cpu(), a[1])
+    _close(b[2], a[2], 1e-5, "weights")
+    _close(b[0], a[0], 2e-5, "experts")
 
 
 @pytest.mark.parametrize("dt", DTYPES)
