@@ -3,12 +3,15 @@ public API of LSaldyt/JAX_llama (reference ``jax_llama/__init__.py:4-10``), plus
 family (Zavevik: gated delta rule + biased attention + table-routed experts) and a third (Zasevik: latent attention
 with a softmax sink + dense / score-routed feed-forwards) and a fourth (Besulix: matrix memories + block-local rotary
 attention beside a time-mix recurrence) and a fifth (Zifisun: windowed latent / normed attention, grouped routing with
-identity experts, several residual streams) on the same layer-list step function.
+identity experts, several residual streams), a sixth (Fokisun: rotary, latent and running-memory layers averaged over the
+depth) and a seventh (Zopupel: differential attention, attention whose values are its keys, norms on both sides of every
+sublayer) on the same layer-list step function.
 
 Framework layer: PyTorch-ROCm. Hot path: hand-written HIP kernels (``csrc/kernels``).
 Multi-GPU: one process per GPU, RCCL + a custom xGMI all-reduce. Decode: hipGraph replay.
 """
-from .config import BesulixConfig, LLaMAConfig, ModelArgs, ZasevikConfig, ZavevikConfig, ZifisunConfig, config_from_params, get_preset, swiglu_hidden_size
+from .config import (BesulixConfig, FokisunConfig, LLaMAConfig, ModelArgs, ZasevikConfig, ZavevikConfig, ZifisunConfig,
+                     ZopupelConfig, config_from_params, get_preset, swiglu_hidden_size)
 from .generation import LLaMA
 from .models import (CausalLMOutput, FlaxLLaMAForCausalLM, FlaxLLaMAModel, KVCache, LLaMAForCausalLM,
                      LLaMAModel)
@@ -18,6 +21,8 @@ from .models.registry import load_model
 from .models.zasevik import ZasevikForCausalLM
 from .models.besulix import BesulixForCausalLM
 from .models.zifisun import ZifisunForCausalLM
+from .models.fokisun import FokisunForCausalLM
+from .models.zopupel import ZopupelForCausalLM
 from .models.zavevik import ZavevikForCausalLM
 from .runtime.engine import GenerationConfig
 from .runtime.stepper import SequenceStepper
@@ -32,5 +37,7 @@ __all__ = [
     "CausalLMOutput", "KVCache", "GenerationConfig",
     "Mesh", "P", "PartitionSpec", "get_llama_param_partition_spec", "with_named_sharding_constraint",
     "with_sharding_constraint", "LLaMA2Tokenizer", "LLaMA3Tokenizer", "ChatFormat", "convert_llama_weights",
-    "ZavevikConfig", "ZavevikForCausalLM", "ZasevikConfig", "ZasevikForCausalLM", "BesulixConfig", "BesulixForCausalLM", "ZifisunConfig", "ZifisunForCausalLM", "SequenceStepper", "load_model",
+    "ZavevikConfig", "ZavevikForCausalLM", "ZasevikConfig", "ZasevikForCausalLM", "BesulixConfig", "BesulixForCausalLM",
+    "ZifisunConfig", "ZifisunForCausalLM", "FokisunConfig", "FokisunForCausalLM", "ZopupelConfig", "ZopupelForCausalLM",
+    "SequenceStepper", "load_model",
 ]
