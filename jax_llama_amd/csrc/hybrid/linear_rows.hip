@@ -15,6 +15,7 @@
 //    g' = min(g, limit), u' = clamp(u).
 //  * an optional per-row scale multiplies the activation row while it is staged (before the operand is rounded): the
 //    input-weighted experts of a score-routed mixture.
+//  * two linears of a few rows can share a launch (a mixture's experts beside its shared expert).
 // The table router's counting sort is here too.
 #include "hy_util.h"
 #include "hybrid.h"
