@@ -47,11 +47,11 @@ the same mechanisms with other values.
   SharedExpertMoE : gated experts chosen by a biased softmax router (weights over the chosen logits), a shared expert.
   SandwichChainBlock : the sandwich-norm residual in one kernel per sublayer, which also leaves the next sublayer's input.
 
-The mixers of the last group split into ``features(proj, ctx, out)`` -- everything between the fused input projection
-``w_in`` and the output matrix ``w_o`` -- so that their block can fuse other rows (a router) into the input product and run
-one output product over the features of all of its members.
-The blocks of the group before the last two split a sublayer into ``features(h, ctx, out=None, gain=1.0)`` (everything up to the output
-projection; ``out`` a column slice to write into, ``gain`` a scalar folded into the last elementwise step) and the
+The mixers of the last two groups split into ``features(proj, ctx, out)`` -- everything between the fused input projection
+``w_in`` and the output matrix ``w_o`` -- so that their block can fuse other rows (a router) into the input product, run one
+output product over the features of all of its members, or choose the features' number format.
+The members of ``SideBySide`` and ``PreNormBlock`` split into ``features(h, ctx, out=None, gain=1.0)`` (everything up to the
+output projection; ``out`` a column slice to write into, ``gain`` a scalar folded into the last elementwise step) and the
 matrix ``w_o``, so a block can fuse the projection with the residual add and ``SideBySide`` can run one projection for
 all of its members.
 """
